@@ -1,5 +1,6 @@
 """Typed configurations and the architecture registry."""
 from .batasun import BatasunConfig
+from .derosun import DerosunConfig
 from .duperax import DuperaxConfig
 from .errors import ConfigError, UnsupportedArchitecture
 from .gemma3 import Gemma3Config
@@ -8,7 +9,7 @@ from .nulunex import NulunexConfig
 from .registry import (Architecture, architectures, find_architecture, load_config,
                        read_config_json, register_architecture)
 from .rilenex import RilenexConfig
-from .spec import (RglruSpec, StreamMixSpec, AttentionSpec, BiasedAttentionSpec, LatentAttentionSpec, Mamba2Spec, RoutedFfnSpec, ScoreBiasSpec, DenseFfnSpec, FeedForwardSpec, GatedDeltaSpec, GatedFfnSpec, Hgrn2Spec, LayerSpec,
+from .spec import (RglruSpec, StreamMixSpec, AttentionSpec, BiasedAttentionSpec, LatentAttentionSpec, Mamba2Spec, MlstmSpec, RoutedFfnSpec, ScoreBiasSpec, DenseFfnSpec, FeedForwardSpec, GatedDeltaSpec, GatedFfnSpec, Hgrn2Spec, LayerSpec,
                    MixerSpec, ModelSpec, NormSpec, ParallelMixerSpec, PositionSpec, RunEntry, TalkingAttentionSpec)
 
 register_architecture(Architecture(
@@ -47,8 +48,14 @@ register_architecture(Architecture(
     parse=NulunexConfig.from_dict,
     spec=lambda cfg, names=None: cfg.model_spec(names)))
 
+register_architecture(Architecture(
+    name=DerosunConfig.architecture,
+    model_types=("derosun",),
+    parse=DerosunConfig.from_dict,
+    spec=lambda cfg, names=None: cfg.model_spec(names)))
+
 __all__ = [
-    "NulunexConfig", "DuperaxConfig", "RglruSpec", "StreamMixSpec", "ConfigError", "UnsupportedArchitecture", "Gemma3Config", "RilenexConfig", "GusedraConfig", "BatasunConfig", "LatentAttentionSpec", "Mamba2Spec", "BiasedAttentionSpec", "RoutedFfnSpec", "ScoreBiasSpec", "Architecture", "architectures",
+    "DerosunConfig", "MlstmSpec", "NulunexConfig", "DuperaxConfig", "RglruSpec", "StreamMixSpec", "ConfigError", "UnsupportedArchitecture", "Gemma3Config", "RilenexConfig", "GusedraConfig", "BatasunConfig", "LatentAttentionSpec", "Mamba2Spec", "BiasedAttentionSpec", "RoutedFfnSpec", "ScoreBiasSpec", "Architecture", "architectures",
     "find_architecture", "load_config", "read_config_json", "register_architecture",
     "AttentionSpec", "FeedForwardSpec", "GatedFfnSpec", "LayerSpec", "MixerSpec", "ModelSpec",
     "NormSpec", "PositionSpec", "RunEntry", "TalkingAttentionSpec", "GatedDeltaSpec", "Hgrn2Spec",

@@ -29,7 +29,7 @@ class NormSpec:
 @dataclass(frozen=True)
 class PositionSpec:
     """A position encoding applied to queries and keys inside a mixer."""
-    kind: str                      # "rope" | "rope_yarn" | "none"
+    kind: str                      # "rope" | "rope_yarn" | "rope_banded" | "none"
     rotary_dim: int = 0
     theta: float = 0.0
     factor: float = 1.0            # linear scaling: positions are divided by it
@@ -43,6 +43,13 @@ class PositionSpec:
     yarn_fast: float = 32.0
     yarn_slow: float = 1.0
     yarn_magnitude_slope: float = 0.1
+    # "rope_banded": a pair whose wavelength l = 2 pi / f is below band_original / band_high keeps its frequency f, above
+    # band_original / band_low it becomes f / band_factor, and between the two, with
+    # s = (band_original / l - band_low) / (band_high - band_low), (1 - s) f / band_factor + s f
+    band_factor: float = 1.0
+    band_low: float = 1.0
+    band_high: float = 4.0
+    band_original: int = 0
 
 
 @dataclass(frozen=True)
@@ -293,6 +300,34 @@ class RglruSpec(MixerSpec):
 
 
 @dataclass(frozen=True)
+class MlstmSpec(MixerSpec):
+    """The matrix memory of xLSTM (state S [heads, v_head_dim, head_dim], n [heads, head_dim] and m [heads]).
+
+    ``q = q_proj x * head_dim^-1/2``, ``k = k_proj x``, ``v = v_proj x``; per head, with cap(z) = gate_cap tanh(z / gate_cap),
+    a log input gate ``i = cap(i_gate x + i_bias)`` and a log forget gate ``f = logsigmoid(cap(f_gate x + f_bias))``;
+    ``m' = max(f + m, i)`` from m = 0; ``S <- exp(f + m - m') S + exp(i - m') k v^T``, n likewise with k alone;
+    ``o = S^T q / (max(|n . q|, exp(-m')) + floor_eps)``; each head's o divided by its root mean square, times ``out_norm``,
+    times ``sigmoid(gate_proj x)``; ``o_proj``."""
+    hidden: int = 0
+    n_heads: int = 0
+    head_dim: int = 0              # queries and keys
+    v_head_dim: int = 0
+    gate_cap: float = 15.0
+    floor_eps: float = 1e-6
+    norm_eps: float = 1e-5         # of the read-out's norm
+    q_proj: str = ""
+    k_proj: str = ""
+    v_proj: str = ""
+    gate_proj: str = ""            # [heads * v_head_dim, hidden]
+    i_gate: str = ""               # [heads, hidden]
+    i_bias: str = ""               # [heads]
+    f_gate: str = ""
+    f_bias: str = ""
+    out_norm: str = ""             # [heads * v_head_dim]
+    o_proj: str = ""
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec(MixerSpec):
     """Mixers side by side on the same input; the result is the sum of ``scales[i] * branches[i]``."""
     branches: Tuple[MixerSpec, ...] = ()
@@ -381,6 +416,8 @@ class LayerSpec:
                     h += post_ffn_norm(ffn(pre_ffn_norm(h)))
     ``"prenorm"``:  the same without the two post norms.
     ``"postnorm"``: h += post_mixer_norm(mixer(h));  h += post_ffn_norm(ffn(h)): the sublayers read the stream itself.
+    ``"postnorm_sum"``: h <- post_mixer_norm(residual_scale h + mixer(h)) and the same with the feed-forward: the norm is
+                    behind the residual sum and replaces the stream.
     ``"streams"``:  the residual is ``ModelSpec.streams`` rows x_1 .. x_S per token; a sublayer reads
                     u = sum_s read[s] x_s, computes y = sublayer(pre_norm(u)), and writes, all streams at once,
                     x_t <- sum_s mix[s, t] x_s + write[t] y (``mixer_streams``, ``ffn_streams``).
@@ -394,6 +431,7 @@ class LayerSpec:
     post_ffn_norm: Optional[NormSpec] = None
     mixer_streams: Optional["StreamMixSpec"] = None
     ffn_streams: Optional["StreamMixSpec"] = None
+    residual_scale: float = 1.0    # "postnorm_sum": the factor on the stream in the sum
 
 
 @dataclass(frozen=True)

@@ -40,12 +40,16 @@ extern "C" int agave_embed_scale(int dtype, const int* tokens, const void* table
 //   r = rows ? rows[i] : i                       (row of h and of branch)
 //   if branch: h[r] += post_gain ? rmsnorm(branch[r]) * post_gain : branch[r]
 //   if out:    out[i] = pre_gain ? rmsnorm(h[r]) * pre_gain : h[r]      (a layer without a norm in front of a sublayer)
+// OF_SUM, the norm behind the residual sum instead of on the branch:
+//   h[r] = rmsnorm(alpha * h[r] + branch[r] + bias) * post_gain      (bias may be null)
 // Gains are 32-bit and already hold the "+1" where the architecture has it.
-template <typename T>
+struct OfSum { float alpha; const float* bias; };
+template <typename T, bool OF_SUM>
 __global__ void residual_norm_kernel(float* __restrict__ h, const T* __restrict__ branch, long ldb, int n_parts,
                                      long part_stride, const float* __restrict__ post_gain, float post_eps,
                                      T* __restrict__ out, long ldo, const float* __restrict__ pre_gain,
-                                     float pre_eps, const int* __restrict__ rows, int e, const float* __restrict__ h_src) {
+                                     float pre_eps, const int* __restrict__ rows, int e, const float* __restrict__ h_src,
+                                     OfSum sum) {
     __shared__ float red[16];
     const int i = blockIdx.x;
     const int r = rows ? rows[i] : i;
@@ -63,18 +67,24 @@ __global__ void residual_norm_kernel(float* __restrict__ h, const T* __restrict_
             return v;
         };
         float inv = 1.0f;
+        auto whole = [&](int c) { return fmaf(sum.alpha, hs[c], at(c) + (sum.bias ? sum.bias[c] : 0.f)); };
         if (post_gain) {
             float ss = 0.f;
             for (int c = threadIdx.x; c < e; c += blockDim.x) {
-                const float v = at(c);
+                const float v = OF_SUM ? whole(c) : at(c);
                 ss += v * v;
             }
             ss = block_sum(ss, red);
             inv = 1.0f / sqrtf(ss / (float)e + post_eps);
         }
         for (int c = threadIdx.x; c < e; c += blockDim.x) {
-            const float y = post_gain ? at(c) * inv * post_gain[c] : at(c);
-            const float hv = hs[c] + y;
+            float hv;
+            if (OF_SUM) {
+                hv = whole(c) * inv * post_gain[c];
+            } else {
+                const float y = post_gain ? at(c) * inv * post_gain[c] : at(c);
+                hv = hs[c] + y;
+            }
             hr[c] = hv;
             ss_h += hv * hv;
         }
@@ -125,18 +135,29 @@ template <> __device__ __forceinline__ void store4<bf16>(bf16* p, float4 v) {
 // loaded is touched before everything has been asked for, so the loads travel together.
 __device__ __forceinline__ float sumsq(bool in, float4 v) { return in ? v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w : 0.f; }
 
-template <typename T, int VPT, int PB>          // PB: slices asked for at a time
+template <typename T, int VPT, int PB, bool OF_SUM>          // PB: slices asked for at a time
 __global__ void residual_norm_fast_kernel(float* __restrict__ h, const T* __restrict__ branch, long ldb, int n_parts,
                                           long part_stride, const float* __restrict__ post_gain, float post_eps,
                                           T* __restrict__ out, long ldo, const float* __restrict__ pre_gain,
                                           float pre_eps, const int* __restrict__ rows, int e,
-                                          const float* __restrict__ h_src) {
+                                          const float* __restrict__ h_src, OfSum sum) {
     __shared__ float red[16];
     const int i = blockIdx.x;
     const int r = rows ? rows[i] : i;
     float* hr = h + (size_t)r * e;
     const float* hs = h_src ? h_src + (size_t)r * e : hr;        // where the row is read (it is always written to h)
     const float4 z = float4{0.f, 0.f, 0.f, 0.f};
+    float4 bias[VPT];
+    if (OF_SUM && sum.bias) {
+#pragma unroll
+        for (int v = 0; v < VPT; ++v) {
+            const int c = (threadIdx.x + v * blockDim.x) * 4;
+            bias[v] = *reinterpret_cast<const float4*>(sum.bias + (c < e ? c : 0));
+        }
+    } else {
+#pragma unroll
+        for (int v = 0; v < VPT; ++v) bias[v] = z;
+    }
     float4 hv[VPT], bv[VPT], g1[VPT], g2[VPT], pv[PB][VPT];
     int col[VPT];
     bool in[VPT];
@@ -180,7 +201,27 @@ __global__ void residual_norm_fast_kernel(float* __restrict__ h, const T* __rest
             }
         }
     }
-    if (branch) {
+    if (branch && OF_SUM) {
+        float ss = 0.f;
+#pragma unroll
+        for (int v = 0; v < VPT; ++v) {
+            hv[v].x = fmaf(sum.alpha, hv[v].x, bv[v].x + bias[v].x);
+            hv[v].y = fmaf(sum.alpha, hv[v].y, bv[v].y + bias[v].y);
+            hv[v].z = fmaf(sum.alpha, hv[v].z, bv[v].z + bias[v].z);
+            hv[v].w = fmaf(sum.alpha, hv[v].w, bv[v].w + bias[v].w);
+            ss += sumsq(in[v], hv[v]);
+        }
+        ss = block_sum(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)e + post_eps);
+#pragma unroll
+        for (int v = 0; v < VPT; ++v) {
+            hv[v].x *= inv * g1[v].x;
+            hv[v].y *= inv * g1[v].y;
+            hv[v].z *= inv * g1[v].z;
+            hv[v].w *= inv * g1[v].w;
+            if (in[v]) *reinterpret_cast<float4*>(hr + col[v]) = hv[v];
+        }
+    } else if (branch) {
         float inv = 1.0f;
         if (post_gain) {
             float ss = 0.f;
@@ -230,13 +271,13 @@ __global__ void residual_norm_fast_kernel(float* __restrict__ h, const T* __rest
     }
 }
 
-template <typename T>
+template <typename T, bool OF_SUM>
 static bool launch_residual_norm_fast(float* h, const void* branch, long ldb, int n_parts, long part_stride,
                                       const float* post_gain, float post_eps,
                                       void* out, long ldo, const float* pre_gain, float pre_eps, const int* rows,
-                                      int n_rows, int e, const float* h_src, hipStream_t stream) {
+                                      int n_rows, int e, const float* h_src, const OfSum& sum, hipStream_t stream) {
     const size_t align = sizeof(T) * 4;
-    if ((uintptr_t)h_src % 16 != 0) return false;
+    if ((uintptr_t)h_src % 16 != 0 || (uintptr_t)sum.bias % 16 != 0) return false;
     if (e % 4 != 0 || e > 16384 || (branch && (ldb % 4 != 0 || (uintptr_t)branch % (n_parts ? 16 : align) != 0)) ||
         (n_parts && part_stride % 4 != 0) ||
         (out && (ldo % 4 != 0 || (uintptr_t)out % align != 0)) || (uintptr_t)h % 16 != 0 ||
@@ -256,13 +297,13 @@ static bool launch_residual_norm_fast(float* h, const void* branch, long ldb, in
     // more than four slices (the output product's runs of heads): eight at a time when a thread holds one float4 of each
 #define RN_FAST(V)                                                                                                    \
     if (n_parts > 4 && V == 1)                                                                                        \
-        residual_norm_fast_kernel<T, V, 8><<<n_rows, threads, 0, stream>>>(h, (const T*)branch, ldb, n_parts,        \
-                                                                           part_stride, post_gain, post_eps, (T*)out, \
-                                                                           ldo, pre_gain, pre_eps, rows, e, h_src);   \
+        residual_norm_fast_kernel<T, V, 8, OF_SUM><<<n_rows, threads, 0, stream>>>(                                   \
+            h, (const T*)branch, ldb, n_parts, part_stride, post_gain, post_eps, (T*)out, ldo, pre_gain, pre_eps,     \
+            rows, e, h_src, sum);                                                                                     \
     else                                                                                                              \
-    residual_norm_fast_kernel<T, V, 4><<<n_rows, threads, 0, stream>>>(h, (const T*)branch, ldb, n_parts, part_stride,  \
-                                                                    post_gain, post_eps,                             \
-                                                                    (T*)out, ldo, pre_gain, pre_eps, rows, e, h_src)
+        residual_norm_fast_kernel<T, V, 4, OF_SUM><<<n_rows, threads, 0, stream>>>(                                   \
+            h, (const T*)branch, ldb, n_parts, part_stride, post_gain, post_eps, (T*)out, ldo, pre_gain, pre_eps,     \
+            rows, e, h_src, sum)
     if (vpt <= 1) RN_FAST(1);
     else if (vpt <= 2) RN_FAST(2);
     else RN_FAST(4);
@@ -274,36 +315,52 @@ static bool launch_residual_norm_fast(float* h, const void* branch, long ldb, in
 // whose sum is the branch (whatever dtype says, which then names out's type alone).
 // h_src: the rows are read there instead of from h (and written to h as ever): the residual stream
 // as a kernel left it that could not write it in place.
+template <bool OF_SUM>
+static int launch_residual_norm(const char* what, int dtype, float* h, const void* branch, long ldb, int n_parts, long part_stride,
+                                const float* post_gain, float post_eps, void* out, long ldo, const float* pre_gain,
+                                float pre_eps, const int* rows, int n_rows, int e, const float* h_src, const OfSum& sum,
+                                hipStream_t stream) {
+    AGAVE_CHECK(n_rows >= 0 && e > 0, "%s: bad sizes rows=%d e=%d", what, n_rows, e);
+    AGAVE_CHECK(h != nullptr, "%s: residual stream is null", what);
+    AGAVE_CHECK(!(h_src && rows), "%s: rows are gathered from the residual stream itself, not from another source", what);
+    AGAVE_CHECK(!branch || ldb >= e, "%s: branch row stride %ld < %d", what, ldb, e);
+    AGAVE_CHECK(!out || ldo >= e, "%s: output row stride %ld < %d", what, ldo, e);
+    AGAVE_CHECK(!(rows && branch), "%s: row gather with a branch is not supported", what);
+    AGAVE_CHECK(n_parts >= 0 && n_parts <= 64 && (n_parts == 0 || branch), "%s: %d slices", what, n_parts);
+    if (n_rows == 0 || (!branch && !out)) return 0;
+    const int threads = e >= 2048 ? 512 : (e >= 512 ? 256 : 64);
+    if (dtype == AGAVE_F32) {
+        if (!launch_residual_norm_fast<float, OF_SUM>(h, branch, ldb, n_parts, part_stride, post_gain, post_eps, out, ldo, pre_gain,
+                                                      pre_eps, rows, n_rows, e, h_src, sum, stream))
+            residual_norm_kernel<float, OF_SUM><<<n_rows, threads, 0, stream>>>(h, (const float*)branch, ldb, n_parts, part_stride,
+                post_gain, post_eps, (float*)out, ldo, pre_gain, pre_eps, rows, e, h_src, sum);
+    } else if (dtype == AGAVE_BF16) {
+        if (!launch_residual_norm_fast<bf16, OF_SUM>(h, branch, ldb, n_parts, part_stride, post_gain, post_eps, out, ldo, pre_gain,
+                                                     pre_eps, rows, n_rows, e, h_src, sum, stream))
+            residual_norm_kernel<bf16, OF_SUM><<<n_rows, threads, 0, stream>>>(h, (const bf16*)branch, ldb, n_parts, part_stride,
+                post_gain, post_eps, (bf16*)out, ldo, pre_gain, pre_eps, rows, e, h_src, sum);
+    } else {
+        AGAVE_CHECK(false, "%s: unknown dtype %d", what, dtype);
+    }
+    AGAVE_LAUNCH_CHECK(what);
+    return 0;
+}
+
 extern "C" int agave_residual_norm(int dtype, float* h, const void* branch, long ldb, int n_parts, long part_stride,
                                    const float* post_gain, float post_eps, void* out, long ldo, const float* pre_gain,
                                    float pre_eps, const int* rows, int n_rows, int e, const float* h_src,
                                    hipStream_t stream) {
-    AGAVE_CHECK(n_rows >= 0 && e > 0, "residual_norm: bad sizes rows=%d e=%d", n_rows, e);
-    AGAVE_CHECK(h != nullptr, "residual_norm: residual stream is null");
-    AGAVE_CHECK(!(h_src && rows), "residual_norm: rows are gathered from the residual stream itself, not from another source");
-    AGAVE_CHECK(!branch || ldb >= e, "residual_norm: branch row stride %ld < %d", ldb, e);
-    AGAVE_CHECK(!out || ldo >= e, "residual_norm: output row stride %ld < %d", ldo, e);
-    AGAVE_CHECK(!(rows && branch), "residual_norm: row gather with a branch is not supported");
-    AGAVE_CHECK(n_parts >= 0 && n_parts <= 64 && (n_parts == 0 || branch), "residual_norm: %d slices", n_parts);
-    if (n_rows == 0 || (!branch && !out)) return 0;
-    const int threads = e >= 2048 ? 512 : (e >= 512 ? 256 : 64);
-    if (dtype == AGAVE_F32 && launch_residual_norm_fast<float>(h, branch, ldb, n_parts, part_stride, post_gain, post_eps,
-                                                              out, ldo, pre_gain, pre_eps, rows, n_rows, e, h_src, stream)) {
-    } else if (dtype == AGAVE_BF16 && launch_residual_norm_fast<bf16>(h, branch, ldb, n_parts, part_stride, post_gain,
-                                                                     post_eps, out, ldo, pre_gain, pre_eps, rows, n_rows,
-                                                                     e, h_src, stream)) {
-    } else if (dtype == AGAVE_F32)
-        residual_norm_kernel<float><<<n_rows, threads, 0, stream>>>(h, (const float*)branch, ldb, n_parts, part_stride,
-                                                                    post_gain, post_eps,
-                                                                    (float*)out, ldo, pre_gain, pre_eps, rows, e, h_src);
-    else if (dtype == AGAVE_BF16)
-        residual_norm_kernel<bf16><<<n_rows, threads, 0, stream>>>(h, (const bf16*)branch, ldb, n_parts, part_stride,
-                                                                   post_gain, post_eps,
-                                                                   (bf16*)out, ldo, pre_gain, pre_eps, rows, e, h_src);
-    else
-        AGAVE_CHECK(false, "residual_norm: unknown dtype %d", dtype);
-    AGAVE_LAUNCH_CHECK("residual_norm");
-    return 0;
+    return launch_residual_norm<false>("residual_norm", dtype, h, branch, ldb, n_parts, part_stride, post_gain, post_eps, out, ldo,
+                                       pre_gain, pre_eps, rows, n_rows, e, h_src, OfSum{1.f, nullptr}, stream);
+}
+
+// h = rmsnorm(alpha * h + branch + bias) * gain;  if out: out = pre_gain ? rmsnorm(h) * pre_gain : h
+extern "C" int agave_norm_of_sum(int dtype, float* h, const void* branch, long ldb, int n_parts, long part_stride, float alpha,
+                                 const float* bias, const float* gain, float eps, void* out, long ldo, const float* pre_gain,
+                                 float pre_eps, int n_rows, int e, hipStream_t stream) {
+    AGAVE_CHECK(branch && gain, "norm_of_sum: a branch and a gain are needed");
+    return launch_residual_norm<true>("norm_of_sum", dtype, h, branch, ldb, n_parts, part_stride, gain, eps, out, ldo, pre_gain,
+                                      pre_eps, nullptr, n_rows, e, nullptr, OfSum{alpha, bias}, stream);
 }
 
 // ------------------------------------------------------------------ residual + layer norms

@@ -111,15 +111,33 @@ extern "C" int agave_embed_scale_packed(const int* tokens, const void* P, float 
 // gelu with the tanh approximation is a = 2 sqrt(2/pi), b = 0.044715 a, limit infinite, shift 0 (0.5 (1 + tanh t) =
 // sigmoid(2t)); silu is a = 1, b = 0; the clamped swish has a limit and shift 1.  The host hands a and b over times
 // -log2(e).  The hardware's exp2 and reciprocal (about an ulp each) stand for the library's functions, whose many
-// instructions a product's last step has no time for.
-struct GateForm { float a, b, limit, shift; };
+// instructions a product's last step has no time for.  gate_b, up_b: vectors added to the two before all of this (one
+// value per output column; both or neither).
+struct GateForm { float a, b, limit, shift; const float *gate_b, *up_b; };
 __device__ __forceinline__ float gated(float gate, float up, const GateForm& F) {
     const float g = fminf(gate, F.limit), u = fminf(fmaxf(up, -F.limit), F.limit);
     const float e = __builtin_amdgcn_exp2f(g * fmaf(F.b, g * g, F.a));
     return g * __builtin_amdgcn_rcpf(1.0f + e) * (u + F.shift);
 }
-static GateForm gate_form(float a, float b, float limit, float shift) {
-    return GateForm{-1.4426950408889634f * a, -1.4426950408889634f * b, limit, shift};
+// the same for output column n of the N there are
+__device__ __forceinline__ float gated_at(float gate, float up, const GateForm& F, int n, int N) {
+    if (F.gate_b) {
+        const int c = n < N ? n : N - 1;
+        gate += F.gate_b[c];
+        up += F.up_b[c];
+    }
+    return gated(gate, up, F);
+}
+static GateForm gate_form(float a, float b, float limit, float shift, const float* gate_b, const float* up_b) {
+    return GateForm{-1.4426950408889634f * a, -1.4426950408889634f * b, limit, shift, gate_b, up_b};
+}
+// the form for a part of the output that starts at column n
+static GateForm from_column(GateForm F, int n) {
+    if (F.gate_b) {
+        F.gate_b += n;
+        F.up_b += n;
+    }
+    return F;
 }
 
 // R: row blocks (of 16 weight rows) per workgroup; MT: tiles of 16 tokens; EPI 0: store, 1: gated;
@@ -276,8 +294,8 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const bf16* __rest
                 if (n + e < N) st(Y + (size_t)m * ldy + n + e, s[e]);
         } else {
             const int n = (nb0 + r) * 8 + g * 2;      // N counts output columns (ff)
-            if (n < N) st(Y + (size_t)m * ldy + n, gated(s[0], s[2], F));
-            if (n + 1 < N) st(Y + (size_t)m * ldy + n + 1, gated(s[1], s[3], F));
+            if (n < N) st(Y + (size_t)m * ldy + n, gated_at(s[0], s[2], F, n, N));
+            if (n + 1 < N) st(Y + (size_t)m * ldy + n + 1, gated_at(s[1], s[3], F, n + 1, N));
         }
     }
 }
@@ -613,8 +631,8 @@ __global__ __launch_bounds__(512) void gemm_row_normed_kernel(RowNorm nz, const 
                 if (n + e < N) st(Y + n + e, s[e]);
         } else {
             const int n = nb * 8 + g * 2;                 // N counts output columns (ff)
-            if (n < N) st(Y + n, gated(s[0], s[2], F));
-            if (n + 1 < N) st(Y + n + 1, gated(s[1], s[3], F));
+            if (n < N) st(Y + n, gated_at(s[0], s[2], F, n, N));
+            if (n + 1 < N) st(Y + n + 1, gated_at(s[1], s[3], F, n + 1, N));
         }
     }
 }
@@ -645,7 +663,7 @@ extern "C" int agave_gemm_row_normed_ok(int M, int N, int K, int epilogue) {
 // going to h_out (see RowNorm).  branch null: Y = pre(h_in) W^T, nothing else is written.
 extern "C" int agave_gemm_row_normed(const float* h_in, float* h_out, const void* branch, int branch_f32, int n_parts,
                                      long part_stride, const float* post_gain, float post_eps, const float* pre_gain,
-                                     float pre_eps, const void* Wp, void* Y, int N, int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift,
+                                     float pre_eps, const void* Wp, void* Y, int N, int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, const float* gate_b, const float* up_b,
                                      hipStream_t stream) {
     AGAVE_CHECK(epilogue == 0 || epilogue == 1, "gemm_row_normed: unknown epilogue %d", epilogue);
     AGAVE_CHECK(agave_gemm_row_normed_ok(1, N, K, epilogue),
@@ -684,7 +702,7 @@ extern "C" int agave_gemm_row_normed(const float* h_in, float* h_out, const void
     else if (K <= 4096) rc = launch_row_normed<EPI_, 2, 8>(nz, Wp, Y, N, K, KB, NB, wgs, lds, F, stream);              \
     else if (!many) rc = launch_row_normed<EPI_, 3, 2>(nz, Wp, Y, N, K, KB, NB, wgs, lds, F, stream);                  \
     else rc = launch_row_normed<EPI_, 3, 8>(nz, Wp, Y, N, K, KB, NB, wgs, lds, F, stream)
-    const GateForm F = gate_form(act_a, act_b, act_limit, act_shift);
+    const GateForm F = gate_form(act_a, act_b, act_limit, act_shift, gate_b, up_b);
     if (epilogue == 1) {
         RN_CASE(1);
     } else {
@@ -708,7 +726,7 @@ extern "C" int agave_gemm_skinny_slices(int M, int N, int K) {
 // and whoever reads Y adds the slices up (a product with few row blocks and many columns then
 // has workgroups enough to keep the memory busy).
 extern "C" int agave_gemm_skinny(const void* X, long ldx, const void* Wp, int dt_y, void* Y, long ldy, int M, int N,
-                                 int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, int splits, hipStream_t stream) {
+                                 int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, const float* gate_b, const float* up_b, int splits, hipStream_t stream) {
     AGAVE_CHECK(M >= 0 && M <= 64 && N > 0 && K > 0, "gemm_skinny: bad sizes M=%d N=%d K=%d (M <= 64)", M, N, K);
     AGAVE_CHECK(K % 8 == 0 && ldx % 8 == 0 && ((uintptr_t)X % 16) == 0,
                 "gemm_skinny: X must be 16-byte aligned with K and its row stride multiples of 8 (K=%d ldx=%ld)", K, ldx);
@@ -727,7 +745,7 @@ extern "C" int agave_gemm_skinny(const void* X, long ldx, const void* Wp, int dt
         else AGAVE_CHECK(false, "gemm_skinny: unknown output dtype %d", dt_y);
     } else {
         AGAVE_CHECK(dt_y == AGAVE_BF16, "gemm_skinny: the gated epilogue writes bfloat16");
-        rc = dispatch_skinny<1, bf16>(X, ldx, Wp, Y, ldy, M, N, K, KB, NB, 1, gate_form(act_a, act_b, act_limit, act_shift), stream);
+        rc = dispatch_skinny<1, bf16>(X, ldx, Wp, Y, ldy, M, N, K, KB, NB, 1, gate_form(act_a, act_b, act_limit, act_shift, gate_b, up_b), stream);
     }
     if (rc != 0) return rc;
     AGAVE_LAUNCH_CHECK("gemm_skinny");
@@ -1244,7 +1262,8 @@ __global__ __launch_bounds__(NWV * 64, 2) void gemm_tiled_kernel(const bf16* __r
                     if (EPI == 0) {
                         store4(reinterpret_cast<TC*>(dst), float4{s0, s1, s2, s3});
                     } else {
-                        const float v0 = gated(s0, s2, F), v1 = gated(s1, s3, F);
+                        const int n = n_base + tile * 8 + (r4 >> 1);
+                        const float v0 = gated_at(s0, s2, F, n, N), v1 = gated_at(s1, s3, F, n + 1, N);
                         *reinterpret_cast<uint32_t*>(dst) = f32x2_to_bf16x2(v0, v1);
                     }
                 }
@@ -1396,9 +1415,9 @@ static int dispatch_tiled(const void* X, long ldx, const void* Wp, void* Y, long
             if (rest <= 64 && (rows16 - rows_main) * 2 * ((M + 127) / 128) <= 256)
                 return launch_tiled<2, 2, 3, EPI, TC, 8, 128, false>(X, ldx, (const uint4*)Wp + w_tile(nb_main, 0, NB, KB) * 64,
                                                                      (TC*)Y + n_main, ldy, M, N - n_main, K, KB, NB - nb_main,
-                                                                     F, stream, 1, 0, NB);
+                                                                     from_column(F, n_main), stream, 1, 0, NB);
             return launch_tiled<2, 2, 3, EPI, TC, 8, 256, false>(X, ldx, (const uint4*)Wp + w_tile(nb_main, 0, NB, KB) * 64,
-                                                                 (TC*)Y + n_main, ldy, M, N - n_main, K, KB, NB - nb_main, F, stream,
+                                                                 (TC*)Y + n_main, ldy, M, N - n_main, K, KB, NB - nb_main, from_column(F, n_main), stream,
                                                                  1, 0, NB);
         }
     }
@@ -1549,7 +1568,7 @@ static int launch_tile_shape(int tile, const void* X, long ldx, const void* Wp, 
 }
 
 extern "C" int agave_gemm_tiled_as(const void* X, long ldx, const void* Wp, int dt_y, void* Y, long ldy, int M, int N,
-                                   int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, int tile, hipStream_t stream) {
+                                   int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, const float* gate_b, const float* up_b, int tile, hipStream_t stream) {
     AGAVE_CHECK(M > 0 && N > 0 && K > 0 && tile >= 0 && tile <= 3, "gemm_tiled_as: bad sizes M=%d N=%d K=%d or tile %d", M, N, K, tile);
     AGAVE_CHECK(K % 8 == 0 && ldx % 8 == 0 && ((uintptr_t)X % 16) == 0,
                 "gemm_tiled_as: X must be 16-byte aligned with K and its row stride multiples of 8 (K=%d ldx=%ld)", K, ldx);
@@ -1559,7 +1578,7 @@ extern "C" int agave_gemm_tiled_as(const void* X, long ldx, const void* Wp, int 
     const int KB = (K + 31) / 32;
     const int NB = epilogue == 0 ? (N + 15) / 16 : (N + 7) / 8;
     int rc;
-    if (epilogue == 1) rc = launch_tile_shape<1, bf16>(tile, X, ldx, Wp, Y, ldy, M, N, K, KB, NB, gate_form(act_a, act_b, act_limit, act_shift), stream);
+    if (epilogue == 1) rc = launch_tile_shape<1, bf16>(tile, X, ldx, Wp, Y, ldy, M, N, K, KB, NB, gate_form(act_a, act_b, act_limit, act_shift, gate_b, up_b), stream);
     else if (dt_y == AGAVE_BF16) rc = launch_tile_shape<0, bf16>(tile, X, ldx, Wp, Y, ldy, M, N, K, KB, NB, GateForm{}, stream);
     else rc = launch_tile_shape<0, float>(tile, X, ldx, Wp, Y, ldy, M, N, K, KB, NB, GateForm{}, stream);
     if (rc != 0) return rc;
@@ -1571,7 +1590,7 @@ extern "C" int agave_gemm_tiled_as(const void* X, long ldx, const void* Wp, int 
 // optional buffer of part_elems floats for partial sums (products with few tiles and many columns
 // are then shared out along the columns); null: never.
 extern "C" int agave_gemm_tiled(const void* X, long ldx, const void* Wp, int dt_y, void* Y, long ldy, int M, int N,
-                                int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, float* part, long part_elems, hipStream_t stream) {
+                                int K, int epilogue, float act_a, float act_b, float act_limit, float act_shift, const float* gate_b, const float* up_b, float* part, long part_elems, hipStream_t stream) {
     AGAVE_CHECK(M >= 0 && N > 0 && K > 0, "gemm_tiled: bad sizes M=%d N=%d K=%d", M, N, K);
     AGAVE_CHECK(K % 8 == 0 && ldx % 8 == 0 && ((uintptr_t)X % 16) == 0,
                 "gemm_tiled: X must be 16-byte aligned with K and its row stride multiples of 8 (K=%d ldx=%ld)", K, ldx);
@@ -1588,7 +1607,7 @@ extern "C" int agave_gemm_tiled(const void* X, long ldx, const void* Wp, int dt_
         else AGAVE_CHECK(false, "gemm_tiled: unknown output dtype %d", dt_y);
     } else {
         AGAVE_CHECK(dt_y == AGAVE_BF16, "gemm_tiled: the gated epilogue writes bfloat16");
-        rc = dispatch_tiled<1, bf16>(X, ldx, Wp, Y, ldy, M, N, K, KB, NB, nullptr, 0, gate_form(act_a, act_b, act_limit, act_shift), stream);
+        rc = dispatch_tiled<1, bf16>(X, ldx, Wp, Y, ldy, M, N, K, KB, NB, nullptr, 0, gate_form(act_a, act_b, act_limit, act_shift, gate_b, up_b), stream);
     }
     if (rc != 0) return rc;
     AGAVE_LAUNCH_CHECK("gemm_tiled");

@@ -17,7 +17,8 @@
 //   latent_turn_queries  the queries' trailing elements rotated, rows to rows or in place;
 //   gate_rows        rows times the sigmoid of 32-bit logits, in place.
 //
-// A rotation turns the first 2 * half of its elements, in pairs (e, e + half) or (2e, 2e + 1).  Angles are made in double
+// A rotation turns the first 2 * half of its elements, in pairs (e, e + half) or (2e, 2e + 1), and multiplies the turned
+// pairs by a magnitude (1 where it is a pure rotation).  Angles are made in double
 // (trig.h); sines, norm sums and the products' sums are 32-bit; T is the element type of the rows between products.
 #include "common_impl.h"
 #include "mfma.h"
@@ -27,15 +28,15 @@
 
 #define MAX_TURNED 256           // pairs a rotation turns at most (their sines wait in LDS)
 
-struct Turn { const double* freq; int half; int neighbours; };       // neighbours: pairs (2e, 2e + 1)
+struct Turn { const double* freq; int half; int neighbours; float magnitude; };     // neighbours: pairs (2e, 2e + 1)
 
 // the sines and cosines of position `pos`, by the threads that share cs (a barrier is the caller's)
 __device__ __forceinline__ void turn_table(const Turn& R, int pos, float (*cs)[MAX_TURNED], int tid, int n_threads) {
     for (int i = tid; i < R.half; i += n_threads) {
         float s, c;
         sincos_of_angle((double)pos * R.freq[i], s, c);
-        cs[0][i] = c;
-        cs[1][i] = s;
+        cs[0][i] = c * R.magnitude;
+        cs[1][i] = s * R.magnitude;
     }
 }
 __device__ __forceinline__ int first_of_pair(const Turn& R, int i) { return R.neighbours ? 2 * i : i; }
@@ -161,11 +162,11 @@ static int check_kv(const char* what, const LatentKv& K, int dtype) {
 // q_heads 0: qraw is a query latent of q_rank; > 0: query rows of q_heads x (q_dim + rot_dim)
 extern "C" int agave_latent_prepare(int dtype, const float* qraw, long ldq, const float* qw, void* qout, long ldqo, int q_rank,
                                     int q_heads, int q_dim, const float* kvraw, long ldkv, const float* kvw, void* krow, long ldkr,
-                                    int kv_rank, int rot_dim, const double* freq, int half, int neighbours, void* k_pages,
+                                    int kv_rank, int rot_dim, const double* freq, int half, int neighbours, float magnitude, void* k_pages,
                                     void* v_pages, const int* table, int width, const int* base, int n_pages, int packed,
                                     const int* tok_seq, const int* tok_pos, int n_tokens, float eps, hipStream_t stream) {
     AGAVE_CHECK(n_tokens >= 0 && (qraw || kvraw) && tok_pos, "latent_prepare: bad sizes N=%d or nothing to prepare", n_tokens);
-    const Turn R{freq, half, neighbours};
+    const Turn R{freq, half, neighbours, magnitude};
     if (check_turn("latent_prepare", R, rot_dim)) return -1;
     const LatentQ Q{qraw, ldq, qw, qout, ldqo, q_rank, q_heads, q_dim, rot_dim};
     if (qraw) {
@@ -191,10 +192,10 @@ __global__ __launch_bounds__(256) void latent_turn_queries_kernel(LatentQ Q, Tur
 
 // rows of the activations' type; q_out may be q (in place)
 extern "C" int agave_latent_turn_queries(int dtype, const void* q, long ldq, void* q_out, long ldqo, int heads, int dim, int rot_dim,
-                                         const double* freq, int half, int neighbours, const int* tok_pos, int n_tokens, hipStream_t stream) {
+                                         const double* freq, int half, int neighbours, float magnitude, const int* tok_pos, int n_tokens, hipStream_t stream) {
     AGAVE_CHECK(n_tokens >= 0 && heads > 0 && dim >= 0 && rot_dim >= 0 && dim + rot_dim > 0 && q && q_out && tok_pos, "latent_turn_queries: bad sizes or buffers");
     AGAVE_CHECK(ldq >= (long)heads * (dim + rot_dim) && ldqo >= (long)heads * (dim + rot_dim) && (q != q_out || ldq == ldqo), "latent_turn_queries: bad row strides");
-    const Turn R{freq, half, neighbours};
+    const Turn R{freq, half, neighbours, magnitude};
     if (check_turn("latent_turn_queries", R, rot_dim)) return -1;
     if (n_tokens == 0) return 0;
     const LatentQ Q{q, ldq, nullptr, q_out, ldqo, 0, heads, dim, rot_dim};
@@ -337,6 +338,8 @@ __device__ __forceinline__ void heads_product_tile(const HeadsProductArgs& A, in
             const float u = ld(r + p), v = ld(r + q);
             float sn, cn;
             sincos_of_angle((double)A.tok_pos[t] * R.freq[e], sn, cn);
+            sn *= R.magnitude;
+            cn *= R.magnitude;
             o[p] = f32_to_bf16(u * cn - v * sn);
             o[q] = f32_to_bf16(v * cn + u * sn);
         }
@@ -384,9 +387,9 @@ static bool heads_product_on_matrix_cores(int dtype, int x_f32, const HeadsProdu
 }
 
 extern "C" int agave_heads_product(int dtype, int x_f32, const void* x, long ldx, int xs, const void* w, void* y, long ldy, int ys,
-                                   const float* gate, long ldg, const double* freq, int half, int neighbours, int tail,
+                                   const float* gate, long ldg, const double* freq, int half, int neighbours, float magnitude, int tail,
                                    const int* tok_pos, int n_tokens, int heads, int n_out, int K, int plain, hipStream_t stream) {
-    HeadsProductArgs A{x, ldx, xs, w, y, ldy, ys, gate, ldg, Turn{freq, half, neighbours}, tail, tok_pos, n_tokens, heads, n_out, K};
+    HeadsProductArgs A{x, ldx, xs, w, y, ldy, ys, gate, ldg, Turn{freq, half, neighbours, magnitude}, tail, tok_pos, n_tokens, heads, n_out, K};
     if (check_heads_product(A)) return -1;
     if (n_tokens == 0) return 0;
     if (!plain && heads_product_on_matrix_cores(dtype, x_f32, A)) {
@@ -415,10 +418,10 @@ extern "C" int agave_latent_decode_rows_ok(int n_tokens, int dim, int rot_dim, i
 // key/value rows into their pages.  q and kvraw are 32-bit rows of the first product.
 extern "C" int agave_latent_decode_rows(const float* q, long ldq, const void* fold, void* folded, long ldf, int heads, int dim,
                                         const float* kvraw, long ldkv, const float* kvw, void* krow, long ldkr, int kv_rank, int rot_dim,
-                                        const double* freq, int half, int neighbours, void* k_pages, void* v_pages, const int* table,
+                                        const double* freq, int half, int neighbours, float magnitude, void* k_pages, void* v_pages, const int* table,
                                         int width, const int* base, int n_pages, int packed, const int* tok_seq, const int* tok_pos,
                                         int n_tokens, float eps, hipStream_t stream) {
-    const Turn R{freq, half, neighbours};
+    const Turn R{freq, half, neighbours, magnitude};
     HeadsProductArgs A{q, ldq, dim + rot_dim, fold, folded, ldf, kv_rank + rot_dim, nullptr, 0, R, rot_dim, tok_pos, n_tokens, heads, kv_rank, dim};
     const LatentKv K{kvraw, ldkv, kvw, krow, ldkr, kv_rank, rot_dim, k_pages, v_pages, table, width, base, n_pages, packed, tok_seq};
     if (check_heads_product(A) || check_turn("latent_decode_rows", R, rot_dim) || check_kv("latent_decode_rows", K, AGAVE_BF16)) return -1;

@@ -12,14 +12,14 @@ from .kernels import _F, _I, _L, _P
 kernels.register_signatures("gemm_mfma", {
     "agave_pack_w16": [_P, _L, _P, _I, _I, _I, _I, _P],
     "agave_embed_scale_packed": [_P, _P, _F, _P, _I, _I, _I, _P],
-    "agave_gemm_skinny": [_P, _L, _P, _I, _P, _L, _I, _I, _I, _I, _F, _F, _F, _F, _I, _P],
+    "agave_gemm_skinny": [_P, _L, _P, _I, _P, _L, _I, _I, _I, _I, _F, _F, _F, _F, _P, _P, _I, _P],
     "agave_gemm_skinny_slices": [_I, _I, _I],
     "agave_gemm_row_normed_ok": [_I, _I, _I, _I],
-    "agave_gemm_row_normed": [_P, _P, _P, _I, _I, _L, _P, _F, _P, _F, _P, _P, _I, _I, _I, _F, _F, _F, _F, _P],
+    "agave_gemm_row_normed": [_P, _P, _P, _I, _I, _L, _P, _F, _P, _F, _P, _P, _I, _I, _I, _F, _F, _F, _F, _P, _P, _P],
     "agave_gemm_tiled_slices": [_I, _I, _I],
     "agave_gemm_tiled_in_slices": [_P, _L, _P, _P, _I, _I, _I, _I, _P],
-    "agave_gemm_tiled": [_P, _L, _P, _I, _P, _L, _I, _I, _I, _I, _F, _F, _F, _F, _P, _L, _P],
-    "agave_gemm_tiled_as": [_P, _L, _P, _I, _P, _L, _I, _I, _I, _I, _F, _F, _F, _F, _I, _P],
+    "agave_gemm_tiled": [_P, _L, _P, _I, _P, _L, _I, _I, _I, _I, _F, _F, _F, _F, _P, _P, _P, _L, _P],
+    "agave_gemm_tiled_as": [_P, _L, _P, _I, _P, _L, _I, _I, _I, _I, _F, _F, _F, _F, _P, _P, _I, _P],
     "agave_gemm_tiled_in_slices_as": [_P, _L, _P, _P, _I, _I, _I, _I, _I, _P],
     "agave_oproj_combine_heads_per_run": [_I, _I, _I, _I],
     "agave_gemm_oproj_combine": [_P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
@@ -29,12 +29,25 @@ SKINNY_MAX_M = 64
 
 
 class GateForm(NamedTuple):
-    """What a product of interleaved gate and up rows ends in: with g = min(gate, limit) and
-    u = clamp(up, -limit, limit), g sigmoid(a g + b g^3) (u + shift)."""
+    """What a product of interleaved gate and up rows ends in: with g = min(gate + gate_bias, limit) and
+    u = clamp(up + up_bias, -limit, limit), g sigmoid(a g + b g^3) (u + shift).  The biases are float32 vectors on the
+    device, one value per output column (both or neither)."""
     a: float
     b: float = 0.0
     limit: float = math.inf
     shift: float = 0.0
+    gate_bias: Optional[torch.Tensor] = None
+    up_bias: Optional[torch.Tensor] = None
+
+    def arguments(self, n_out: int) -> tuple:
+        """As the entry points take it, for a product of ``n_out`` output columns."""
+        if (self.gate_bias is None) != (self.up_bias is None):
+            raise ValueError("a gated product has a bias on gate and up or on neither")
+        for b in (self.gate_bias, self.up_bias):
+            if b is not None:
+                kernels._dev(b)
+                kernels._f32vec(b, "gated product's bias", n_out)
+        return (self.a, self.b, self.limit, self.shift, kernels.ptr(self.gate_bias), kernels.ptr(self.up_bias))
 
 
 GELU_TANH = GateForm(2.0 * math.sqrt(2.0 / math.pi), 2.0 * math.sqrt(2.0 / math.pi) * 0.044715)     # 0.5 (1 + tanh t) = sigmoid(2 t)
@@ -142,7 +155,7 @@ def row_normed(h_in: torch.Tensor, h_out: Optional[torch.Tensor], branch: Option
     library.call(kernels.lib("gemm_mfma"), "agave_gemm_row_normed", h_in.data_ptr(), kernels.ptr(h_out), kernels.ptr(branch),
                  1 if (branch is not None and branch.dtype == torch.float32) else 0, n_parts, part_stride,
                  kernels.ptr(post_gain), post_eps, pre_gain.data_ptr(), pre_eps, packed.data_ptr(), out.data_ptr(),
-                 n_out, k, epilogue, *form, kernels.stream())
+                 n_out, k, epilogue, *form.arguments(n_out), kernels.stream())
 
 
 _slices = {}
@@ -209,7 +222,7 @@ def tiled_as(x: torch.Tensor, packed: torch.Tensor, out: torch.Tensor, n_out: in
     if packed.numel() != nb * ((k + 31) // 32) * 512:
         raise ValueError("packed product: the packed weight does not fit these sizes")
     library.call(kernels.lib("gemm_mfma"), "agave_gemm_tiled_as", x.data_ptr(), x.stride(0), packed.data_ptr(),
-                 kernels.dt(out), out.data_ptr(), out.stride(0), m, n_out, k, epilogue, *form, tile, kernels.stream())
+                 kernels.dt(out), out.data_ptr(), out.stride(0), m, n_out, k, epilogue, *form.arguments(n_out), tile, kernels.stream())
 
 
 def tiled_slices_as(x: torch.Tensor, packed: torch.Tensor, out: torch.Tensor, n_out: int, tile: int) -> None:
@@ -238,7 +251,7 @@ def skinny_slices(x: torch.Tensor, packed: torch.Tensor, out: torch.Tensor, n_ou
     if packed.numel() != ((n_out + 15) // 16) * ((k + 31) // 32) * 512:
         raise ValueError("packed product: the packed weight does not fit these sizes")
     library.call(kernels.lib("gemm_mfma"), "agave_gemm_skinny", x.data_ptr(), x.stride(0), packed.data_ptr(),
-                 kernels.dt(out), out.data_ptr(), n_out, m, n_out, k, 0, *NO_FORM, out.shape[0], kernels.stream())
+                 kernels.dt(out), out.data_ptr(), n_out, m, n_out, k, 0, *NO_FORM.arguments(n_out), out.shape[0], kernels.stream())
 
 
 # The tiled kernel shares a product out along its columns only when it has fewer than 160 tiles of
@@ -274,11 +287,11 @@ def _launch(fn: str, x: torch.Tensor, packed: torch.Tensor, out: torch.Tensor, n
     if fn == "agave_gemm_tiled":
         part = _partial_sums(x, epilogue)
         library.call(kernels.lib("gemm_mfma"), fn, x.data_ptr(), x.stride(0), packed.data_ptr(),
-                     kernels.dt(out), out.data_ptr(), out.stride(0), m, n_out, k, epilogue, *form,
+                     kernels.dt(out), out.data_ptr(), out.stride(0), m, n_out, k, epilogue, *form.arguments(n_out),
                      kernels.ptr(part), part.numel() if part is not None else 0, kernels.stream())
         return
     library.call(kernels.lib("gemm_mfma"), fn, x.data_ptr(), x.stride(0), packed.data_ptr(),
-                 kernels.dt(out), out.data_ptr(), out.stride(0), m, n_out, k, epilogue, *form, 1, kernels.stream())
+                 kernels.dt(out), out.data_ptr(), out.stride(0), m, n_out, k, epilogue, *form.arguments(n_out), 1, kernels.stream())
 
 
 def try_linear(x: torch.Tensor, lin, out: torch.Tensor) -> bool:

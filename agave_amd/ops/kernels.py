@@ -22,6 +22,7 @@ _SIGNATURES = {
     "elementwise": {
         "agave_embed_scale": [_I, _P, _P, _F, _P, _I, _I, _I, _P],
         "agave_residual_norm": [_I, _P, _P, _L, _I, _L, _P, _F, _P, _L, _P, _F, _P, _I, _I, _P, _P],
+        "agave_norm_of_sum": [_I, _P, _P, _L, _I, _L, _F, _P, _P, _F, _P, _L, _P, _F, _I, _I, _P],
         "agave_residual_layernorm": [_I, _P, _P, _L, _I, _L, _P, _P, _F, _P, _L, _P, _P, _F, _P, _I, _I, _P, _P],
         "agave_qk_norm_rope_kv": [_I, _P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _F, _F, _P, _I, _F,
                                   _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
@@ -176,6 +177,37 @@ def residual_norm(h: torch.Tensor, branch: Optional[torch.Tensor], post_gain: Op
             raise TypeError("branch and out must have the same dtype")
     library.call(lib("elementwise"), "agave_residual_norm", dt(act), ptr(h), ptr(branch), ldb, n_parts, part_stride,
                  ptr(post_gain), post_eps, ptr(out), ldo, ptr(pre_gain), pre_eps, ptr(rows), n, e, ptr(src), stream())
+
+
+def norm_of_sum(h: torch.Tensor, branch: torch.Tensor, alpha: float, bias: Optional[torch.Tensor], gain: torch.Tensor, eps: float,
+                out: Optional[torch.Tensor] = None, pre_gain: Optional[torch.Tensor] = None, pre_eps: float = 0.0) -> None:
+    """h = rmsnorm(alpha * h + branch + bias) * gain, the norm behind the residual sum (``bias`` may be None; ``branch`` as in
+    :func:`residual_norm`).  If ``out``: out = rmsnorm(h) * pre_gain, or the rows of h rounded to ``out``'s type where
+    ``pre_gain`` is None."""
+    _dev(h, branch, bias, gain, out, pre_gain)
+    if h.dtype != torch.float32 or h.dim() != 2 or not h.is_contiguous():
+        raise ValueError("residual stream must be a contiguous float32 [rows, hidden] tensor")
+    n, e = h.shape
+    for v, what in ((bias, "bias"), (gain, "gain"), (pre_gain, "pre_gain")):
+        _f32vec(v, what, e)
+    ldo = n_parts = part_stride = 0
+    if branch.dim() == 3:
+        if branch.dtype != torch.float32 or branch.shape[1:] != (n, e) or not branch.is_contiguous():
+            raise ValueError(f"partial sums must be a contiguous float32 [slices, {n}, {e}] tensor")
+        n_parts, part_stride, ldb = branch.shape[0], n * e, e
+    else:
+        ldb = _rows(branch, "branch")
+        if branch.shape != (n, e):
+            raise ValueError(f"branch must be [{n}, {e}], got {tuple(branch.shape)}")
+    if out is not None:
+        ldo = _rows(out, "out")
+        if out.shape != (n, e):
+            raise ValueError(f"out must be [{n}, {e}], got {tuple(out.shape)}")
+        if n_parts == 0 and branch.dtype != out.dtype:
+            raise TypeError("branch and out must have the same dtype")
+    library.call(lib("elementwise"), "agave_norm_of_sum", dt(out if out is not None else branch), ptr(h), ptr(branch), ldb, n_parts,
+                 part_stride, float(alpha), ptr(bias), ptr(gain), float(eps), ptr(out), ldo, ptr(pre_gain), float(pre_eps), n, e,
+                 stream())
 
 
 def residual_layernorm(h: torch.Tensor, branch: Optional[torch.Tensor], post_w: Optional[torch.Tensor],

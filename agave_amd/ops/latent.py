@@ -21,15 +21,15 @@ MAX_SPLITS = 64          # workgroups that share a row's pages at most
 MAX_PAIRS = 256          # pairs a rotation turns at most
 
 kernels.register_signatures(LIBRARY, {
-    "agave_latent_prepare": [_I, _P, _L, _P, _P, _L, _I, _I, _I, _P, _L, _P, _P, _L, _I, _I, _P, _I, _I, _P, _P, _P, _I, _P, _I, _I,
+    "agave_latent_prepare": [_I, _P, _L, _P, _P, _L, _I, _I, _I, _P, _L, _P, _P, _L, _I, _I, _P, _I, _I, _F, _P, _P, _P, _I, _P, _I, _I,
                              _P, _P, _I, _F, _P],
-    "agave_latent_turn_queries": [_I, _P, _L, _P, _L, _I, _I, _I, _P, _I, _I, _P, _I, _P],
+    "agave_latent_turn_queries": [_I, _P, _L, _P, _L, _I, _I, _I, _P, _I, _I, _F, _P, _I, _P],
     "agave_latent_decode_rows_ok": [_I, _I, _I, _I],
-    "agave_latent_decode_rows": [_P, _L, _P, _P, _L, _I, _I, _P, _L, _P, _P, _L, _I, _I, _P, _I, _I, _P, _P, _P, _I, _P, _I, _I, _P, _P,
+    "agave_latent_decode_rows": [_P, _L, _P, _P, _L, _I, _I, _P, _L, _P, _P, _L, _I, _I, _P, _I, _I, _F, _P, _P, _P, _I, _P, _I, _I, _P, _P,
                                  _I, _F, _P],
     "agave_latent_fresh_pages": [_P, _L, _I, _P, _L, _I, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "agave_gate_rows": [_I, _P, _L, _P, _L, _I, _I, _P],
-    "agave_heads_product": [_I, _I, _P, _L, _I, _P, _P, _L, _I, _P, _L, _P, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P],
+    "agave_heads_product": [_I, _I, _P, _L, _I, _P, _P, _L, _I, _P, _L, _P, _I, _I, _F, _I, _P, _I, _I, _I, _I, _I, _P],
 })
 kernels.register_signatures(ATTENTION, {
     "agave_latent_decode_ok": [_I, _I, _I, _I],
@@ -41,6 +41,7 @@ kernels.register_signatures(ATTENTION, {
 class Turn(NamedTuple):
     freq: Optional[torch.Tensor]         # float64 [pairs], or None: nothing is turned
     neighbours: bool = False             # pairs (2e, 2e + 1) instead of (e, e + pairs)
+    magnitude: float = 1.0               # multiplies sine and cosine
 
 
 NO_TURN = Turn(None)
@@ -136,7 +137,7 @@ def latent_prepare(step, eps: float, turn: Turn, rot_dim: int, *, q_raw: Optiona
         _i32(step.tok_seq, "sequences", n)
     library.call(_lib(), "agave_latent_prepare", dt(some), ptr(q_raw), ldq, ptr(q_weight), ptr(q_out), ldqo, q_rank, q_heads, q_dim,
                  ptr(kv_raw), ldkv, ptr(kv_weight), ptr(k_row), ldkr, kv_rank, rot_dim, ptr(turn.freq), half,
-                 1 if turn.neighbours else 0, *page_args, ptr(step.tok_seq), ptr(step.tok_pos), n, float(eps), stream())
+                 1 if turn.neighbours else 0, float(turn.magnitude), *page_args, ptr(step.tok_seq), ptr(step.tok_pos), n, float(eps), stream())
 
 
 def turn_queries(q: torch.Tensor, q_out: torch.Tensor, n_heads: int, dim: int, rot_dim: int, turn: Turn, tok_pos: torch.Tensor) -> None:
@@ -146,7 +147,7 @@ def turn_queries(q: torch.Tensor, q_out: torch.Tensor, n_heads: int, dim: int, r
     ldq, ldqo = _typed_rows(q, "q", n, cols, q.dtype), _typed_rows(q_out, "q_out", n, cols, q.dtype)
     _i32(tok_pos, "positions", n)
     library.call(_lib(), "agave_latent_turn_queries", dt(q), ptr(q), ldq, ptr(q_out), ldqo, n_heads, dim, rot_dim, ptr(turn.freq),
-                 _turn(turn, rot_dim, "turn_queries"), 1 if turn.neighbours else 0, ptr(tok_pos), n, stream())
+                 _turn(turn, rot_dim, "turn_queries"), 1 if turn.neighbours else 0, float(turn.magnitude), ptr(tok_pos), n, stream())
 
 
 def heads_product(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, n_heads: int, x_head: int, y_head: int, *,
@@ -178,7 +179,7 @@ def heads_product(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, n_heads: in
     if (k + tail) * 4 > 60 * 1024:
         raise ValueError(f"heads_product: a head of {k + tail} input elements is too long")
     library.call(_lib(), "agave_heads_product", dt(y), 1 if x.dtype == torch.float32 else 0, ptr(x), ldx, x_head, ptr(w), ptr(y), ldy,
-                 y_head, ptr(gate), ldg, ptr(turn.freq), half, 1 if turn.neighbours else 0, tail, ptr(tok_pos), n, n_heads, n_out, k,
+                 y_head, ptr(gate), ldg, ptr(turn.freq), half, 1 if turn.neighbours else 0, float(turn.magnitude), tail, ptr(tok_pos), n, n_heads, n_out, k,
                  1 if force_plain else 0, stream())
 
 
@@ -203,7 +204,7 @@ def decode_rows(q_raw: torch.Tensor, fold: torch.Tensor, folded: torch.Tensor, n
     _i32(step.tok_seq, "sequences", n)
     library.call(_lib(), "agave_latent_decode_rows", ptr(q_raw), ldq, ptr(fold), ptr(folded), ldf, n_heads, dim, ptr(kv_raw), ldkv,
                  ptr(kv_weight), None, 0, kv_rank, rot_dim, ptr(turn.freq), _turn(turn, rot_dim, "decode_rows"),
-                 1 if turn.neighbours else 0, *_pages(pages, kd, kv_rank, bf), ptr(step.tok_seq), ptr(step.tok_pos), n, float(eps),
+                 1 if turn.neighbours else 0, float(turn.magnitude), *_pages(pages, kd, kv_rank, bf), ptr(step.tok_seq), ptr(step.tok_pos), n, float(eps),
                  stream())
 
 

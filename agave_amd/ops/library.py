@@ -28,7 +28,7 @@ FLAGS = ["-O3", "-std=c++17", "-shared", "-fPIC", f"--offload-arch={ARCH}",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-command-line-argument"]
 
 LIBRARIES = ("elementwise", "gemm", "gemm_mfma", "attention_plain", "attention_mfma", "attention_biased", "routed_ffn",
-             "sequence", "latent", "attention_latent", "streams", "rglru", "sampling", "peaks")
+             "sequence", "latent", "attention_latent", "streams", "rglru", "mlstm", "sampling", "peaks")
 
 _loaded: Dict[str, ctypes.CDLL] = {}
 _lock = threading.Lock()

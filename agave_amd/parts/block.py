@@ -9,6 +9,11 @@ sublayers read the stream itself, rounded to the activations' type,
 
     h += post_mixer_norm(mixer(h));  h += post_ffn_norm(ffn(h))
 
+``postnorm_sum`` has the norm behind the residual sum, which replaces the stream (Xiong et al., "On Layer Normalization
+in the Transformer Architecture", call this order Post-LN), with a factor on the stream:
+
+    h <- post_mixer_norm(alpha h + mixer(h));  h <- post_ffn_norm(alpha h + ff(h))
+
 A block never adds its last branch
 itself: it returns it as *pending* ``(branch, norm | None)``, and whoever runs next (the
 next block's first norm, or the model's end) hands it to the norm that comes next
@@ -24,7 +29,7 @@ import torch
 from ..config.spec import LayerSpec
 from ..weights.loader import TensorNeed
 from .base import BuildEnv, lookup, register
-from .norm import NormedRows, Pending, add_branch, rows_as_they_are
+from .norm import NormedRows, NormOfSum, Pending, RmsNorm, add_branch, rows_as_they_are
 
 
 NORMED_ROWS_AS_A_PROMISE = 1        # up to this many rows a sublayer may make its normalised input itself
@@ -151,6 +156,21 @@ class PostNormBlock(SandwichBlock):
         return (self.ffn.forward(x, step), self.post_ffn)
 
 
+class PostNormSumBlock(PostNormBlock):
+    """The norm behind the residual sum: the pending branch carries a norm that takes in the stream too.  A feed-forward
+    that ends in a bias leaves it to the kernel that norms."""
+
+    def __init__(self, spec: LayerSpec, weights, env: BuildEnv):
+        super().__init__(spec, weights, env)
+        if not isinstance(self.post_mixer, RmsNorm) or (self.ffn is not None and not isinstance(self.post_ffn, RmsNorm)):
+            raise ValueError("a postnorm_sum block needs an RMS norm behind every sublayer")
+        self.post_mixer = NormOfSum(self.post_mixer, spec.residual_scale)
+        if self.ffn is not None:
+            hand_over = getattr(self.ffn, "hand_over_bias", None)
+            self.post_ffn = NormOfSum(self.post_ffn, spec.residual_scale, hand_over() if hand_over is not None else None)
+
+
 register("block", "sandwich", SandwichBlock)
 register("block", "postnorm", PostNormBlock)
+register("block", "postnorm_sum", PostNormSumBlock)
 register("block", "prenorm", PreNormBlock)

@@ -11,7 +11,7 @@ in 32-bit, the stacked product is followed by the elementwise kernel, which take
 """
 from __future__ import annotations
 
-from typing import List
+from typing import List, Optional
 
 import torch
 
@@ -35,12 +35,12 @@ class GatedFfn:
         self.spec = spec
         self.env = env
         # [gate; up] stacked; on the matrix cores their rows are interleaved so that the product ends in the
-        # activation (where it has such a form, and without a bias on gate or up: the fused product has no place for one)
+        # activation (where it has such a form; biases on both are added inside it)
         def bias(name):
             return weights.get(name) if name else None
 
         form = gemm_mfma.gate_form_of(spec.activation, spec.act_limit, spec.act_alpha)
-        fused = form is not None and not (spec.gate_bias or spec.up_bias)
+        fused = form is not None and bool(spec.gate_bias) == bool(spec.up_bias)
         self.gate_up = Linear([weights.get(spec.gate_proj), weights.get(spec.up_proj)], env, "gate_up",
                               interleave_ff=spec.intermediate if fused else 0,
                               biases=[bias(spec.gate_bias), bias(spec.up_bias)], gate_form=form or gemm_mfma.GELU_TANH)
@@ -56,6 +56,11 @@ class GatedFfn:
             if name:
                 needs.append(TensorNeed(name, (size,)))
         return needs
+
+    def hand_over_bias(self) -> Optional[torch.Tensor]:
+        """The bias of what :meth:`forward` returns, for a block whose next kernel adds it: from now on the result is
+        without it."""
+        return self.down.hand_over_bias()
 
     def forward(self, x: torch.Tensor, step, slices_ok: bool = True, tag: str = "ffn") -> torch.Tensor:
         """``slices_ok`` False: the result is wanted as rows of the activations' type (a caller that is no

@@ -95,13 +95,13 @@ class LatentAttention:
         if s.rot_dim and s.position.kind != "none":
             position = lookup("position", s.position.kind)(s.position, env)
             table = getattr(position, "rotation_table", None)
-            if table is None or getattr(position, "magnitude", 1.0) != 1.0:
-                raise ValueError(f"latent attention: the position encoding {s.position.kind!r} is no plain rotation of pairs")
+            if table is None:
+                raise ValueError(f"latent attention: the position encoding {s.position.kind!r} is no rotation of pairs")
             freq, neighbours = table()
             if freq is not None:
                 if 2 * freq.numel() > s.rot_dim:
                     raise ValueError(f"latent attention: {2 * freq.numel()} rotated elements exceed rot_dim ({s.rot_dim})")
-                self.turn = ops.Turn(freq.contiguous(), neighbours)
+                self.turn = ops.Turn(freq.contiguous(), neighbours, float(getattr(position, "magnitude", 1.0)))
         # decode steps run on kernels of their own where the cached rows' sizes allow (pages in operand order)
         self.decode_ok = env.dtype == torch.bfloat16 and ops.decode_attention_ok(self.kd, s.kv_rank, s.v_head_dim)
 

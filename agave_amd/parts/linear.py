@@ -26,7 +26,8 @@ class Linear:
         ``interleave_ff``: the stack is [gate; up] of that many rows each; if the weight is packed
         its rows are interleaved for the product that ends in ``gate_form`` (see ``forward_gated``).
         ``biases``: one vector [out_i] or None per matrix; y = W x + b then (the sum is made in
-        32-bit by a kernel of its own after the product: a model without biases pays nothing)."""
+        32-bit by a kernel of its own after the product, or inside the gated form where the product
+        ends in one: a model without biases pays nothing)."""
         ws = []
         for w in weights:
             if w.dim() != 2:
@@ -58,8 +59,6 @@ class Linear:
         if biases is not None and any(b is not None for b in biases):
             if len(biases) != len(ws):
                 raise ValueError(f"{name}: {len(biases)} biases for {len(ws)} matrices")
-            if interleave_ff:
-                raise ValueError(f"{name}: a product that ends in a gate's form takes no bias")
             pieces = []
             for w, b in zip(ws, biases):
                 if b is None:
@@ -68,6 +67,9 @@ class Linear:
                     raise ValueError(f"{name}: a bias of shape {tuple(b.shape)} for a matrix of {w.shape[0]} rows")
                 pieces.append(b.to(device=env.device, dtype=torch.float32))
             self.bias = torch.cat(pieces).contiguous()
+            if self.interleave_ff:              # gate and up: inside the form that the product ends in
+                self.gate_form = gate_form._replace(gate_bias=pieces[0].contiguous(), up_bias=pieces[1].contiguous())
+                self.bias = None
 
     def forward(self, x: torch.Tensor, out: Optional[torch.Tensor] = None,
                 out_dtype: Optional[torch.dtype] = None, tag: Optional[str] = None,
@@ -103,6 +105,11 @@ class Linear:
             kernels.add_bias(out, self.bias)
         library.profile.label = None
         return out
+
+    def hand_over_bias(self) -> Optional[torch.Tensor]:
+        """The bias vector (None: there is none), for a caller that adds it itself from now on."""
+        bias, self.bias = self.bias, None
+        return bias
 
     def takes_partials(self, n: int, n_heads: int, head_dim: int, splits: int) -> bool:
         """Whether :meth:`forward_partials` can take the decode attention's partial results for

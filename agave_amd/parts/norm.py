@@ -55,6 +55,7 @@ def add_branch(h: torch.Tensor, pending: Pending) -> None:
     elif isinstance(post, LayerNorm):
         kernels.residual_layernorm(h, branch, post.weight, post.bias, post.eps, None, None, None, 0.0, src=base)
     else:
+        # (other kinds, the norm of the residual sum among them: what they write for themselves)
         if base is not None:
             h.copy_(base)
         post.add_to(h, branch)
@@ -113,6 +114,9 @@ def rows_as_they_are(h: torch.Tensor, pending: Pending, out: torch.Tensor, rows:
     the (chosen) rows of ``h`` are handed on, rounded to ``out``'s element type.  One kernel where the
     branch's norm is an RMS norm (or none) and all rows are wanted, as with a norm in front."""
     branch, post, base = unpack_pending(pending)
+    if isinstance(post, NormOfSum) and base is None and rows is None and (branch.dim() == 3 or branch.dtype == out.dtype):
+        kernels.norm_of_sum(h, branch, post.alpha, post.bias, post.gain, post.eps, out)
+        return
     fused = rows is None and branch is not None and (post is None or isinstance(post, RmsNorm))
     if fused and branch.dim() == 2 and branch.dtype != out.dtype:
         fused = False
@@ -170,6 +174,10 @@ class RmsNorm(Norm):
         """One kernel adds the branch (through the RMS norm after its sublayer, if it has one) and
         computes this norm, reading and writing ``h`` once."""
         branch, post, base = unpack_pending(pending)
+        if isinstance(post, NormOfSum) and out is not None and rows is None and base is None \
+                and (branch.dim() == 3 or branch.dtype == out.dtype):
+            kernels.norm_of_sum(h, branch, post.alpha, post.bias, post.gain, post.eps, out, self.gain, self.eps)
+            return
         if branch is not None and post is not None and not isinstance(post, RmsNorm):
             add_branch(h, (branch, post, base))     # another kind of norm after the sublayer: its own kernel
             branch = post = base = None
@@ -183,6 +191,19 @@ class RmsNorm(Norm):
                               post.eps if (branch is not None and post) else 0.0,
                               out, self.gain if out is not None else None, self.eps if out is not None else 0.0, rows,
                               src=base)
+
+
+class NormOfSum(Norm):
+    """The norm behind the residual sum, ``h <- rms(alpha h + branch + bias) * gain``, as the post norm of a pending branch:
+    an RMS norm's weight and eps, the factor on the stream, and a bias that the branch was left without (None: none).
+    Whoever takes the branch adds it, norms the sum and makes its own rows of it in one kernel."""
+
+    def __init__(self, norm: RmsNorm, alpha: float, bias: Optional[torch.Tensor] = None):
+        self.gain, self.eps, self.size = norm.gain, norm.eps, norm.size
+        self.alpha, self.bias = float(alpha), bias
+
+    def add_to(self, h, branch) -> None:
+        kernels.norm_of_sum(h, branch, self.alpha, self.bias, self.gain, self.eps)
 
 
 class LayerNorm(Norm):

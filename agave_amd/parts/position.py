@@ -73,6 +73,24 @@ class YarnRotaryPosition(RotaryPosition):
         raise ValueError("rope_yarn scales sine and cosine: the q/k kernel of the plain rotation does not apply it")
 
 
+class BandedRotaryPosition(RotaryPosition):
+    """The same rotation with frequencies scaled by wavelength, as Llama 3.1 does: with ``l = 2 pi / f``, pairs with ``l <
+    original / high`` keep f, pairs with ``l > original / low`` get ``f / factor``, those between are blended by ``s = (original
+    / l - low) / (high - low)`` into ``(1 - s) f / factor + s f``.  The frequencies are made in double."""
+
+    def __init__(self, spec: PositionSpec, env: BuildEnv):
+        super().__init__(PositionSpec("rope", rotary_dim=spec.rotary_dim, theta=spec.theta, interleaved=spec.interleaved), env)
+        if spec.band_factor <= 0 or spec.band_original < 1 or spec.band_low <= 0 or spec.band_high <= 0:
+            raise ValueError("rope_banded needs a positive factor, original context, low and high")
+        turns = spec.band_original * self._exact / (2.0 * math.pi)         # original / wavelength
+        slow = self._exact / float(spec.band_factor)
+        width = spec.band_high - spec.band_low
+        s = (turns - spec.band_low) / (width if width != 0.0 else 1.0)
+        blend = (1.0 - s) * slow + s * self._exact
+        self._exact = np.where(turns > spec.band_high, self._exact, np.where(turns < spec.band_low, slow, blend))
+        self.inv_freq = torch.from_numpy(self._exact.astype(np.float32)).to(env.device)
+
+
 class NoPosition:
     def __init__(self, spec: PositionSpec, env: BuildEnv):
         pass
@@ -86,4 +104,5 @@ class NoPosition:
 
 register("position", "rope", RotaryPosition)
 register("position", "rope_yarn", YarnRotaryPosition)
+register("position", "rope_banded", BandedRotaryPosition)
 register("position", "none", NoPosition)
