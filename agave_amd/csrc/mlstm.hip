@@ -110,7 +110,8 @@ __global__ __launch_bounds__(256) void mlstm_step_kernel(MlstmArgs A, float* __r
             else S[u][r][0] = cols[u][dd];
         }
     }
-    const float m1 = fmaxf(f + m0, i), keep = expf(f + m0 - m1), write = expf(i - m1);
+    const double kept = (double)f + (double)m0;              // (in double, so that a small f is not lost beside m)
+    const float m1 = (float)fmax(kept, (double)i), keep = exp_of_difference(kept, m1), write = exp_of_difference(i, m1);
     float kq = 0.f;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
@@ -165,7 +166,7 @@ __global__ __launch_bounds__(256) void mlstm_readout_kernel(MlstmArgs A, const f
     const float* w = A.weight + (long)h * dv;
     float i, f;
     log_gates(A, row, h, i, f);
-    const float m1 = fmaxf(f + A.m[sh], i);
+    const float m1 = (float)fmax((double)f + (double)A.m[sh], (double)i);
     const float inv_den = 1.0f / (fmaxf(fabsf(nq[row * A.nh + h]), expf(-m1)) + A.floor_eps);
     float o[KEEP], ss = 0.f;
 #pragma unroll

@@ -23,7 +23,7 @@ The other published shapes:
 
 Another design beside the closest Gemma 3 shape of equal size (not the default run):
 
-    python bench.py --design rilenex|gusedra|batasun|duperax|nulunex [--design-size small|medium|large] [--design-layers 8]
+    python bench.py --design rilenex|gusedra|batasun|duperax|nulunex|derosun [--design-size small|medium|large] [--design-layers 8]
 
 prints one JSON line with, for that decoder and for a Gemma 3 decoder of the same width, depth,
 heads and about as many weights: tokens a second of a 2,048-token prompt and of decode steps at
@@ -312,6 +312,26 @@ def nulunex_config(size: str, layers: int) -> dict:
     return {"architecture": "Nulunex", "vocab": 32768, "width": e, "norm": {"eps": 1e-5}, "layers": out}
 
 
+def derosun_config(size: str, layers: int) -> dict:
+    """Of every four layers the first and the third are matrix memories in the proportions of the published xLSTM models
+    (heads of 256 keys and 512 values, as many as make the width), the second has attention with whole-row norms, a rotation
+    scaled by wavelength and capped scores, the fourth latent attention with a query latent in the proportions of the
+    Batasun shape beside it (a cached row of 192 + 64 numbers at the small size, 512 + 64 at the others).  Neither
+    attention has a window.  Every layer has a dense feed-forward of two thirds of the inner size, with biases."""
+    e, ff, h, g, d, _, _ = DESIGN_SIZES[size]
+    kv_rank = 192 if size == "small" else 512
+    dense = {"kind": "dense", "ff": (2 * ff // 3) // 256 * 256}
+    memory = {"type": "mlstm", "mixer": {"heads": e // 512, "dim": 256, "vdim": 512, "gate_cap": 15.0}}
+    attention = {"type": "attention",
+                 "mixer": {"heads": h, "kv_heads": g, "dim": d, "vdim": d, "scale": d ** -0.5, "softcap": 30.0,
+                           "rot": {"dims": d, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+    latent = {"type": "latent_attention",
+              "mixer": {"heads": h, "dim": d, "rot_dim": d // 2, "vdim": d, "q_rank": 3 * e // 4, "kv_rank": kv_rank, "scale": (d + d // 2) ** -0.5,
+                        "rot": {"base": 10000.0, "dims": d // 2, "scaling": {"factor": 40.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    return {"architecture": "Derosun", "vocab": 32768, "width": e, "norm": {"eps": 1e-5}, "postln_alpha": 2.0, "embedding": {"scale": 1.0},
+            "layers": [dict((memory, attention, memory, latent)[i % 4], mlp=dense) for i in range(layers)]}
+
+
 def gemma_like_config(size: str, layers: int) -> dict:
     """The same width, depth and heads as a Gemma 3 decoder; its gated feed-forward has three matrices,
     so two thirds of the inner size give as many weights."""
@@ -361,7 +381,7 @@ def compare_designs(args) -> int:
               "dtype": "bf16", "data": "synthetic: uniform-random token ids, random weights", "sizes": DESIGN_SIZES[size],
               "peaks_measured": measured_peaks()}
     makers = {"rilenex": rilenex_config, "gusedra": gusedra_config, "batasun": batasun_config, "duperax": duperax_config,
-              "nulunex": nulunex_config}
+              "nulunex": nulunex_config, "derosun": derosun_config}
     runs = [(args.design, makers[args.design](size, layers))]
     if args.design in ("batasun", "duperax"):      # the design with the same attention kernels and routed feed-forwards stands beside it too
         runs.append(("gusedra_equal_size", gusedra_config(size, layers)))
@@ -369,6 +389,9 @@ def compare_designs(args) -> int:
         runs.append(("rilenex_equal_size", rilenex_config(size, layers)))
     if args.design == "nulunex":                   # the designs with the same latent attention, and with the same attention and feed-forward
         runs += [("batasun_equal_size", batasun_config(size, layers)), ("duperax_equal_size", duperax_config(size, layers))]
+    if args.design == "derosun":                   # recurrent layers and latent attention with a query latent; capped scores; dense feed-forwards
+        runs += [("batasun_equal_size", batasun_config(size, layers)), ("duperax_equal_size", duperax_config(size, layers)),
+                 ("nulunex_equal_size", nulunex_config(size, layers))]
     runs.append(("gemma3_equal_size", gemma_like_config(size, layers)))
     for name, cfg in runs:
         engine = Engine.from_random(cfg, seed=0, dtype="bfloat16", max_slots=batch, max_context=context,
@@ -409,7 +432,7 @@ def main() -> int:
     ap.add_argument("--no-points", action="store_true", help="skip prefill and the batch 1 / 64 points")
     ap.add_argument("--prefill-only", action="store_true",
                     help="time only the 2048-token prefill and print its record (for profiles)")
-    ap.add_argument("--design", choices=["rilenex", "gusedra", "batasun", "duperax", "nulunex"], help="measure this design beside a Gemma 3 decoder of equal size")
+    ap.add_argument("--design", choices=["rilenex", "gusedra", "batasun", "duperax", "nulunex", "derosun"], help="measure this design beside a Gemma 3 decoder of equal size")
     ap.add_argument("--design-size", default="medium", choices=sorted(DESIGN_SIZES))
     ap.add_argument("--design-layers", type=int, default=8)
     args = ap.parse_args()

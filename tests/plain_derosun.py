@@ -89,7 +89,9 @@ def tensor_shapes(cfg: dict) -> Dict[str, tuple]:
 
 def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
     """Weights that keep activations of order one, rounded to bfloat16 values (so that a bfloat16 checkpoint holds exactly
-    these numbers).  The forget gates lean towards remembering, the input gates spread over both signs."""
+    these numbers).  The forget gates lean towards remembering, the input gates spread over both signs.  The matrix memory's
+    queries lean towards its keys: a token's read-out is normed to one, so with q and k unrelated the sign of a product q.k
+    near zero (all that a first token's read-out has of it) would decide over whole rows, and rounding over the sign."""
     g = torch.Generator().manual_seed(seed)
     out = {}
     for name, shape in tensor_shapes(cfg).items():
@@ -107,6 +109,10 @@ def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
         else:
             t = torch.randn(shape, generator=g, dtype=F) / math.sqrt(shape[-1])
         out[name] = t.to(torch.bfloat16).to(F)
+    for i, layer in enumerate(cfg["layers"]):
+        if layer["type"] == "mlstm":
+            p = f"l{i}.mix."
+            out[p + "q"] = (0.9 * out[p + "k"] + 0.45 * out[p + "q"]).to(torch.bfloat16).to(F)
     return out
 
 
@@ -262,20 +268,33 @@ def dense_ff(h, w, p):
 MIXERS = {"attention": "attention", "latent_attention": "latent_attention", "mlstm": "mlstm"}
 
 
-def forward(cfg: dict, weights: Dict[str, torch.Tensor], tokens: Sequence[int], layers_out: Optional[List] = None) -> torch.Tensor:
-    """Logits [T, vocab] of one sequence.  ``layers_out`` receives the residual stream after every layer."""
+def forward(cfg: dict, weights: Dict[str, torch.Tensor], tokens: Sequence[int], layers_out: Optional[List] = None,
+            shake: Optional[torch.Generator] = None) -> torch.Tensor:
+    """Logits [T, vocab] of one sequence.  ``layers_out`` receives the residual stream after every layer.  ``shake``: what a
+    sublayer reads and what it returns is multiplied by 1 + 2^-9 noise, as much as rounding to bfloat16 moves it (see
+    :func:`sensitivity`)."""
+    def s(t):
+        return t if shake is None else t * (1.0 + 2.0 ** -9 * torch.randn(t.shape, generator=shake, dtype=F))
     w = {k: v.to(F) for k, v in weights.items()}
     eps, alpha = cfg["norm"]["eps"], cfg["postln_alpha"]
     x = w["embed"][torch.tensor(list(tokens))] * cfg["embedding"]["scale"]
     for i, layer in enumerate(cfg["layers"]):
         p = f"l{i}."
         mix = globals()[MIXERS[layer["type"]]]
-        x = norm_of_sum(x, mix(x, w, p + "mix.", layer["mixer"], eps), w[p + "norm1"], alpha, eps)
+        x = norm_of_sum(x, s(mix(s(x), w, p + "mix.", layer["mixer"], eps)), w[p + "norm1"], alpha, eps)
         if layer["mlp"] is not None:
-            x = norm_of_sum(x, dense_ff(x, w, p + "mlp."), w[p + "norm2"], alpha, eps)
+            x = norm_of_sum(x, s(dense_ff(s(x), w, p + "mlp.")), w[p + "norm2"], alpha, eps)
         if layers_out is not None:
             layers_out.append(x.clone())
     return (rms(x, eps) * w["final.norm"]) @ w["head"].T
+
+
+def sensitivity(cfg: dict, weights, tokens: Sequence[int], ref: torch.Tensor, runs: int = 6) -> torch.Tensor:
+    """[T]: how far a position's logits move at most when the forward pass is shaken, over some runs.  Most positions move
+    little; where a norm divides a read-out that almost cancels, or a latent of one element stands near zero, they move much,
+    and no computation in bfloat16 can do better there."""
+    g = torch.Generator().manual_seed(len(tokens))
+    return torch.stack([(forward(cfg, weights, tokens, shake=g) - ref).abs().max(-1).values for _ in range(runs)]).max(0).values
 
 
 def argmax_first(row) -> int:
