@@ -29,7 +29,6 @@
 #include <math.h>
 
 #define CHUNK 128
-#define TILE 32                  // tokens a workgroup of mlstm_read takes
 #define KEY_BLOCKS (CHUNK / 16)
 #define MAX_DK 1024
 #define MAX_DV 1024
@@ -207,6 +206,18 @@ __device__ __forceinline__ ChunkPlace chunk_of(const MlstmArgs& A, int s, int c)
     return p;
 }
 
+// What the `per` workgroups of one (chunk, head) read besides their own rows is the same for all of them, and every XCD has
+// an L2 of its own: workgroup ids go round the XCDs, so the ids of a unit's workgroups are XCDS apart.
+#define XCDS 8
+struct UnitPlace { int sub, c, h, s; };          // s < 0: no such unit
+__device__ __forceinline__ UnitPlace unit_of(int id, int per, int chunks, int nh, int n_seqs) {
+    const int unit = id / (XCDS * per) * XCDS + id % XCDS;
+    UnitPlace u{id / XCDS % per, unit % chunks, unit / chunks % nh, unit / (chunks * nh)};
+    if (u.s >= n_seqs) u.s = -1;
+    return u;
+}
+static long unit_workgroups(long units, long per) { return (units + XCDS - 1) / XCDS * XCDS * per; }
+
 __global__ __launch_bounds__(CHUNK) void mlstm_gates_kernel(MlstmArgs A, ChunkArgs C) {
     __shared__ double tot[CHUNK / 64], most[CHUNK / 64];
     const int h = blockIdx.y, s = blockIdx.z, j = threadIdx.x, lane = j & 63, wv = j >> 6;
@@ -245,16 +256,18 @@ __global__ __launch_bounds__(CHUNK) void mlstm_gates_kernel(MlstmArgs A, ChunkAr
 
 // A wave's tile is 64 rows d by 64 columns e of sum_j exp(a_j - top) k_j v_j^T; four waves, four tiles a workgroup.
 template <bool VEC>
-__global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmArgs A, ChunkArgs C, int chunks) {
+__global__ __launch_bounds__(256) void mlstm_chunk_kernel(MlstmArgs A, ChunkArgs C, int chunks, int per) {
     __shared__ float w[CHUNK];
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, c16 = lane & 15, g = lane >> 4;
-    const int h = blockIdx.y, s = blockIdx.z / chunks, dk = A.dk, dv = A.dv;
-    const ChunkPlace P = chunk_of(A, s, blockIdx.z % chunks);
+    const UnitPlace U0 = unit_of(blockIdx.x, per, chunks, A.nh, A.n_seqs);
+    if (U0.s < 0) return;
+    const int h = U0.h, dk = A.dk, dv = A.dv;
+    const ChunkPlace P = chunk_of(A, U0.s, U0.c);
     if (P.count <= 0) return;                                // (the whole workgroup)
     const long nh_at = P.number * A.nh + h;
     if (threadIdx.x < CHUNK) w[threadIdx.x] = exp_of_difference(C.a[nh_at * CHUNK + threadIdx.x], C.top_all[nh_at]);
     __syncthreads();
-    const int tiles_d = (dk + 63) / 64, tiles = tiles_d * ((dv + 63) / 64), tile = (int)blockIdx.x * 4 + wv;
+    const int tiles_d = (dk + 63) / 64, tiles = tiles_d * ((dv + 63) / 64), tile = U0.sub * 4 + wv;
     if (tile >= tiles) return;                               // (no barrier follows)
     const int d0 = (tile % tiles_d) * 64, e0 = (tile / tiles_d) * 64;
     const float *kp[4], *vp[4];
@@ -390,18 +403,20 @@ __global__ __launch_bounds__(256) void mlstm_carry_kernel(MlstmArgs A, ChunkArgs
     if (writer) C.m_end[(long)s * A.nh + h] = m;             // (the state's own m is still read by the other workgroups)
 }
 
-// A workgroup of NW waves has TILE tokens of one chunk and head: the waves share out the keys of the scores, then the columns
-// of the values (EB blocks of 16 each).
-template <typename T, int EB, int NW, bool VEC>
-__global__ __launch_bounds__(NW * 64) void mlstm_read_kernel(MlstmArgs A, ChunkArgs C, T* __restrict__ out, long ldo) {
-    __shared__ __attribute__((aligned(16))) f32x4_t ps[2][KEY_BLOCKS][64];      // weighted scores, as they are made and used
+// A workgroup of NW waves has TT tiles of 16 tokens of one chunk and head: the waves share out the keys of the scores, then the
+// columns of the values (EB blocks of 16 each).
+template <typename T, int TT, int EB, int NW, bool VEC>
+__global__ __launch_bounds__(NW * 64) void mlstm_read_kernel(MlstmArgs A, ChunkArgs C, int chunks, T* __restrict__ out, long ldo) {
+    constexpr int TILE = 16 * TT, PER = CHUNK / TILE;
+    __shared__ __attribute__((aligned(16))) f32x4_t ps[TT][KEY_BLOCKS][64];      // weighted scores, as they are made and used
     __shared__ double a_s[CHUNK], b_s[TILE];
     __shared__ float from_start[TILE], floor_s[TILE], nq_s[TILE], row_part[NW][TILE], ss_part[NW][TILE];
     const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, c16 = lane & 15, g = lane >> 4;
-    const int h = blockIdx.y, s = blockIdx.z, dk = A.dk, dv = A.dv;
-    constexpr int PER = CHUNK / TILE;
-    const ChunkPlace P = chunk_of(A, s, blockIdx.x / PER);
-    const int t0 = (blockIdx.x % PER) * TILE;                // first token of the tile, in the chunk
+    const UnitPlace U = unit_of(blockIdx.x, PER, chunks, A.nh, A.n_seqs);
+    if (U.s < 0) return;
+    const int h = U.h, s = U.s, dk = A.dk, dv = A.dv;
+    const ChunkPlace P = chunk_of(A, s, U.c);
+    const int t0 = U.sub * TILE;                             // first token of the tile, in the chunk
     if (P.count <= t0) return;                               // (the whole workgroup)
     const long nh_at = P.number * A.nh + h, rows0 = P.first;
     const double m0 = (double)C.m0[nh_at];
@@ -415,41 +430,128 @@ __global__ __launch_bounds__(NW * 64) void mlstm_read_kernel(MlstmArgs A, ChunkA
         from_start[tid] = exp_of_difference(m0, b);
         floor_s[tid] = expf(-(float)(C.F[at] + b));
     }
-    // n . q of the starting state: NW * 2 threads a token
+    // n . q of the starting state: NW * 4 / TT threads a token, eight loads of each on their way at a time
     {
-        constexpr int SH = NW * 2;
+        constexpr int SH = NW * 4 / TT, AHEAD = 8;
         const int t = tid / SH, p = tid % SH;
         const float* qr = A.q + (rows0 + min(t0 + t, last)) * A.ld + (long)h * dk;
         const float* nr = start + (long)dv * dk;
         float x = 0.f;
-        for (int d = p; d < dk; d += SH) x = fmaf(qr[d], nr[d], x);
+        for (int d0 = 4 * p; d0 < dk; d0 += 4 * SH * AHEAD) {
+            f32x4_t qx[AHEAD], nx[AHEAD];
+#pragma unroll
+            for (int u = 0; u < AHEAD; ++u) {
+                qx[u] = four<VEC>(qr, d0 + 4 * SH * u, dk);
+                nx[u] = four<VEC>(nr, d0 + 4 * SH * u, dk);
+            }
+#pragma unroll
+            for (int u = 0; u < AHEAD; ++u)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x = fmaf(qx[u][e], nx[u][e], x);
+        }
 #pragma unroll
         for (int off = 1; off < SH; off *= 2) x += __shfl_xor(x, off);
         if (p == 0) nq_s[t] = x;
     }
     // the state behind the step's last token
-    if (blockIdx.x % PER == 0 && tid == 0 && P.first + P.count == A.cu[s + 1])
+    if (U.sub == 0 && tid == 0 && P.first + P.count == A.cu[s + 1])
         A.m[(long)A.slots[s] * A.nh + h] = C.m_end[(long)s * A.nh + h];
     __syncthreads();
-    const float* q0 = A.q + (rows0 + min(t0 + c16, last)) * A.ld + (long)h * dk;
-    const float* q1 = A.q + (rows0 + min(t0 + 16 + c16, last)) * A.ld + (long)h * dk;
+    const float* qp[TT];
+#pragma unroll
+    for (int u = 0; u < TT; ++u) qp[u] = A.q + (rows0 + min(t0 + 16 * u + c16, last)) * A.ld + (long)h * dk;
     const int blocks = (min(t0 + TILE, P.count) + 15) / 16;  // blocks of 16 keys that the tile's tokens see
-    float row_sum[2] = {0.f, 0.f};
+    const int steps = (dk + 15) / 16;                        // a lane takes elements 16 step + 4 g and its three neighbours
+    // this wave's columns of the values are e0 + 16 b + c16 (a wave without columns reads the last one and stores nothing)
+    const int e0 = wv * EB * 16;
+    const float *sp[EB], *vp[EB];
+#pragma unroll
+    for (int b = 0; b < EB; ++b) {
+        const int e = min(e0 + 16 * b + c16, dv - 1);
+        sp[b] = start + (long)e * dk;
+        vp[b] = A.v + rows0 * A.ld + (long)h * dv + e;
+    }
+    // two sets of operands take turns, so that one is on its way while the other is multiplied
+    f32x4_t qf[2][TT], sf[2][EB];
+    auto ask_state = [&](int buf, int step) {
+        const int d = 16 * min(step, steps - 1) + 4 * g;
+#pragma unroll
+        for (int u = 0; u < TT; ++u) qf[buf][u] = four<VEC>(qp[u], d, dk);
+#pragma unroll
+        for (int b = 0; b < EB; ++b) sf[buf][b] = four<VEC>(sp[b], d, dk);
+    };
+    f32x4_t acc[TT][EB];
+#pragma unroll
+    for (int u = 0; u < TT; ++u)
+#pragma unroll
+        for (int b = 0; b < EB; ++b) acc[u][b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    auto use_state = [&](int buf, int step) {
+        if (step >= steps) return;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int b = 0; b < EB; ++b)
+#pragma unroll
+                for (int u = 0; u < TT; ++u) acc[u][b] = mfma_16x16x4(qf[buf][u][r], sf[buf][b][r], acc[u][b]);
+    };
+    float vx[2][4][EB];
+    auto ask_values = [&](int buf, int jb) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const long j = (long)min(16 * min(jb, blocks - 1) + 4 * g + r, last) * A.ld;
+#pragma unroll
+            for (int b = 0; b < EB; ++b) vx[buf][r][b] = vp[b][j];
+        }
+    };
+    auto use_values = [&](int buf, int jb) {
+        if (jb >= blocks) return;
+        f32x4_t pf[TT];
+#pragma unroll
+        for (int u = 0; u < TT; ++u) pf[u] = ps[u][jb][lane];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int b = 0; b < EB; ++b)
+#pragma unroll
+                for (int u = 0; u < TT; ++u) acc[u][b] = mfma_16x16x4(pf[u][r], vx[buf][r][b], acc[u][b]);
+    };
+    float row_sum[TT] = {};
     for (int jb = wv; jb < blocks; jb += NW) {
         const float* kr = A.k + (rows0 + min(16 * jb + c16, last)) * A.ld + (long)h * dk;
-        f32x4_t sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-#pragma unroll 4
-        for (int d = 4 * g; d < (dk + 15) / 16 * 16; d += 16) {
-            const f32x4_t kf = four<VEC>(kr, d, dk), qa = four<VEC>(q0, d, dk), qb = four<VEC>(q1, d, dk);
+        f32x4_t sc[TT];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                sc[0] = mfma_16x16x4(kf[r], qa[r], sc[0]);
-                sc[1] = mfma_16x16x4(kf[r], qb[r], sc[1]);
+        for (int u = 0; u < TT; ++u) sc[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        constexpr int U4 = 4;
+        f32x4_t kf[2][U4], qk[2][U4][TT];
+        auto ask = [&](int buf, int s0) {
+#pragma unroll
+            for (int u = 0; u < U4; ++u) {
+                const int d = 16 * min(s0 + u, steps - 1) + 4 * g;
+                kf[buf][u] = four<VEC>(kr, d, dk);
+#pragma unroll
+                for (int x = 0; x < TT; ++x) qk[buf][u][x] = four<VEC>(qp[x], d, dk);
             }
+        };
+        auto use = [&](int buf, int s0) {
+#pragma unroll
+            for (int u = 0; u < U4; ++u) {
+                if (s0 + u >= steps) break;
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+#pragma unroll
+                    for (int x = 0; x < TT; ++x) sc[x] = mfma_16x16x4(kf[buf][u][r], qk[buf][u][x][r], sc[x]);
+            }
+        };
+        ask(0, 0);
+        for (int s0 = 0; s0 < steps; s0 += 2 * U4) {
+            ask(1, s0 + U4);
+            use(0, s0);
+            ask(0, s0 + 2 * U4);
+            use(1, s0 + U4);
         }
         // the lane holds keys 16 jb + 4 g + r against token t0 + 16 u + c16
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
+        for (int u = 0; u < TT; ++u) {
             const int t = t0 + 16 * u + c16;
             f32x4_t p;
 #pragma unroll
@@ -461,71 +563,51 @@ __global__ __launch_bounds__(NW * 64) void mlstm_read_kernel(MlstmArgs A, ChunkA
             ps[u][jb][lane] = p;
         }
     }
+    ask_state(0, 0);                                         // (on its way across the meeting of the waves)
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
+    for (int u = 0; u < TT; ++u) {
         float x = row_sum[u];
         x += __shfl_xor(x, 16);
         x += __shfl_xor(x, 32);
         if (g == 0) row_part[wv][16 * u + c16] = x;
     }
     __syncthreads();
-    // values: this wave's columns e0 + 16 b + c16
-    const int e0 = wv * EB * 16;
-    f32x4_t acc[2][EB];
+    for (int step = 0; step < steps; step += 2) {
+        ask_state(1, step + 1);
+        use_state(0, step);
+        ask_state(0, step + 2);
+        use_state(1, step + 1);
+    }
+    ask_values(0, 0);
+    // the lane holds tokens 16 u + 4 g + r of the tile
 #pragma unroll
-    for (int b = 0; b < EB; ++b) acc[0][b] = acc[1][b] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    if (e0 < dv) {
-        const float *sp[EB], *vp[EB];
+    for (int u = 0; u < TT; ++u)
 #pragma unroll
-        for (int b = 0; b < EB; ++b) {
-            const int e = min(e0 + 16 * b + c16, dv - 1);
-            sp[b] = start + (long)e * dk;
-            vp[b] = A.v + rows0 * A.ld + (long)h * dv + e;
+        for (int r = 0; r < 4; ++r) {
+            const float x = A.q_scale * from_start[16 * u + 4 * g + r];
+#pragma unroll
+            for (int b = 0; b < EB; ++b) acc[u][b][r] *= x;
         }
-#pragma unroll 2
-        for (int d = 4 * g; d < (dk + 15) / 16 * 16; d += 16) {
-            const f32x4_t qa = four<VEC>(q0, d, dk), qb = four<VEC>(q1, d, dk);
-            f32x4_t sf[EB];
+    for (int jb = 0; jb < blocks; jb += 2) {
+        ask_values(1, jb + 1);
+        use_values(0, jb);
+        ask_values(0, jb + 2);
+        use_values(1, jb + 1);
+    }
+    // what the last step reads, asked for before the waves meet (without conditions, from inside the rows)
+    float gt[TT][4][EB], wt[EB];
 #pragma unroll
-            for (int b = 0; b < EB; ++b) sf[b] = four<VEC>(sp[b], d, dk);
+    for (int b = 0; b < EB; ++b) {
+        const int e = min(e0 + 16 * b + c16, dv - 1);
+        wt[b] = A.weight[(long)h * dv + e];
 #pragma unroll
-            for (int r = 0; r < 4; ++r)
+        for (int u = 0; u < TT; ++u)
 #pragma unroll
-                for (int b = 0; b < EB; ++b) {
-                    acc[0][b] = mfma_16x16x4(qa[r], sf[b][r], acc[0][b]);
-                    acc[1][b] = mfma_16x16x4(qb[r], sf[b][r], acc[1][b]);
-                }
-        }
-        // the lane holds tokens 16 u + 4 g + r of the tile
-#pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const float x = A.q_scale * from_start[16 * u + 4 * g + r];
-#pragma unroll
-                for (int b = 0; b < EB; ++b) acc[u][b][r] *= x;
-            }
-        for (int jb = 0; jb < blocks; ++jb) {
-            const f32x4_t pa = ps[0][jb][lane], pb = ps[1][jb][lane];
-            float vx[4][EB];
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const long j = (long)min(16 * jb + 4 * g + r, last) * A.ld;
-#pragma unroll
-                for (int b = 0; b < EB; ++b) vx[r][b] = vp[b][j];
-            }
-#pragma unroll
-            for (int r = 0; r < 4; ++r)
-#pragma unroll
-                for (int b = 0; b < EB; ++b) {
-                    acc[0][b] = mfma_16x16x4(pa[r], vx[r][b], acc[0][b]);
-                    acc[1][b] = mfma_16x16x4(pb[r], vx[r][b], acc[1][b]);
-                }
-        }
+            for (int r = 0; r < 4; ++r) gt[u][r][b] = A.gate[(rows0 + min(t0 + 16 * u + 4 * g + r, last)) * A.ld + (long)h * dv + e];
     }
     // division and the norm's sum of squares
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int u = 0; u < TT; ++u)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int t = 16 * u + 4 * g + r;
@@ -547,7 +629,7 @@ __global__ __launch_bounds__(NW * 64) void mlstm_read_kernel(MlstmArgs A, ChunkA
         }
     __syncthreads();
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+    for (int u = 0; u < TT; ++u)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int t = 16 * u + 4 * g + r;
@@ -561,8 +643,7 @@ __global__ __launch_bounds__(NW * 64) void mlstm_read_kernel(MlstmArgs A, ChunkA
             for (int b = 0; b < EB; ++b) {
                 const int e = e0 + 16 * b + c16;
                 if (e >= dv) continue;
-                const float gt = A.gate[row * A.ld + (long)h * dv + e];
-                st(out + row * ldo + (long)h * dv + e, acc[u][b][r] * inv * A.weight[(long)h * dv + e] * sigmoid_of(gt));
+                st(out + row * ldo + (long)h * dv + e, acc[u][b][r] * inv * wt[b] * sigmoid_of(gt[u][r][b]));
             }
         }
 }
@@ -622,14 +703,22 @@ extern "C" int agave_mlstm_step(int dtype, const float* q, const float* k, const
 
 extern "C" int agave_mlstm_chunk_size() { return CHUNK; }
 
+// (two tiles of 16 tokens a workgroup read the chunk's starting state half as often; one tile where two would leave
+// compute units idle)
+template <typename T, int TT, bool VEC>
+static void launch_read(const MlstmArgs& A, const ChunkArgs& C, T* out, long ldo, int chunks, hipStream_t stream) {
+    const unsigned grid = (unsigned)unit_workgroups((long)chunks * A.nh * A.n_seqs, CHUNK / (16 * TT));
+    if (A.dv <= 64) mlstm_read_kernel<T, TT, 1, 4, VEC><<<grid, 256, 0, stream>>>(A, C, chunks, out, ldo);
+    else if (A.dv <= 128) mlstm_read_kernel<T, TT, 2, 4, VEC><<<grid, 256, 0, stream>>>(A, C, chunks, out, ldo);
+    else if (A.dv <= 256) mlstm_read_kernel<T, TT, 4, 4, VEC><<<grid, 256, 0, stream>>>(A, C, chunks, out, ldo);
+    else if (A.dv <= 512) mlstm_read_kernel<T, TT, 8, 4, VEC><<<grid, 256, 0, stream>>>(A, C, chunks, out, ldo);
+    else mlstm_read_kernel<T, TT, 8, 8, VEC><<<grid, 512, 0, stream>>>(A, C, chunks, out, ldo);
+}
+
 template <typename T, bool VEC>
-static void launch_read(const MlstmArgs& A, const ChunkArgs& C, T* out, long ldo, int max_rows, hipStream_t stream) {
-    const dim3 grid((max_rows + TILE - 1) / TILE, A.nh, A.n_seqs);
-    if (A.dv <= 64) mlstm_read_kernel<T, 1, 4, VEC><<<grid, 256, 0, stream>>>(A, C, out, ldo);
-    else if (A.dv <= 128) mlstm_read_kernel<T, 2, 4, VEC><<<grid, 256, 0, stream>>>(A, C, out, ldo);
-    else if (A.dv <= 256) mlstm_read_kernel<T, 4, 4, VEC><<<grid, 256, 0, stream>>>(A, C, out, ldo);
-    else if (A.dv <= 512) mlstm_read_kernel<T, 8, 4, VEC><<<grid, 256, 0, stream>>>(A, C, out, ldo);
-    else mlstm_read_kernel<T, 8, 8, VEC><<<grid, 512, 0, stream>>>(A, C, out, ldo);
+static void choose_read(const MlstmArgs& A, const ChunkArgs& C, T* out, long ldo, int chunks, hipStream_t stream) {
+    if ((long)chunks * A.nh * A.n_seqs * (CHUNK / 32) < 256) launch_read<T, 1, VEC>(A, C, out, ldo, chunks, stream);
+    else launch_read<T, 2, VEC>(A, C, out, ldo, chunks, stream);
 }
 
 // gates: double [3][numbers][nh][CHUNK]; totals: double [2][numbers][nh]; m0: float [numbers + n_seqs][nh];
@@ -645,27 +734,28 @@ extern "C" int agave_mlstm_chunks(int dtype, const float* q, const float* k, con
     AGAVE_CHECK(max_rows >= 0 && max_rows <= n_tokens, "mlstm_chunks: a sequence of %d rows in a step of %d", max_rows, n_tokens);
     if (n_tokens == 0 || n_seqs == 0 || max_rows == 0) return 0;
     const int chunks = (max_rows + CHUNK - 1) / CHUNK;
-    AGAVE_CHECK((long)chunks * n_seqs <= 65535, "mlstm_chunks: %d sequences of %d chunks", n_seqs, chunks);
     const long per = numbers * nh;
     const ChunkArgs C{gates, gates + per * CHUNK, gates + 2 * per * CHUNK, totals, totals + per, m0, m0 + per, part};
     const bool vec = by_fours(A) && ((uintptr_t)part % 16) == 0;
     mlstm_gates_kernel<<<dim3(chunks, nh, n_seqs), CHUNK, 0, stream>>>(A, C);
     AGAVE_LAUNCH_CHECK("mlstm_gates");
     const int tiles = ((dk + 63) / 64) * ((dv + 63) / 64);
-    const dim3 grid((tiles + 3) / 4, nh, chunks * n_seqs);
-    if (vec) mlstm_chunk_kernel<true><<<grid, 256, 0, stream>>>(A, C, chunks);
-    else mlstm_chunk_kernel<false><<<grid, 256, 0, stream>>>(A, C, chunks);
+    const int wgs = (tiles + 3) / 4;
+    const long units = (long)chunks * nh * n_seqs;
+    AGAVE_CHECK(unit_workgroups(units, wgs > CHUNK / 16 ? wgs : CHUNK / 16) < (1L << 31), "mlstm_chunks: too many chunks, heads and sequences");
+    if (vec) mlstm_chunk_kernel<true><<<(unsigned)unit_workgroups(units, wgs), 256, 0, stream>>>(A, C, chunks, wgs);
+    else mlstm_chunk_kernel<false><<<(unsigned)unit_workgroups(units, wgs), 256, 0, stream>>>(A, C, chunks, wgs);
     AGAVE_LAUNCH_CHECK("mlstm_chunk");
     const long count = (long)(dv + 1) * dk;
     if (vec) mlstm_carry_kernel<4><<<dim3((unsigned)((count / 4 + 255) / 256), nh, n_seqs), 256, 0, stream>>>(A, C);
     else mlstm_carry_kernel<1><<<dim3((unsigned)((count + 255) / 256), nh, n_seqs), 256, 0, stream>>>(A, C);
     AGAVE_LAUNCH_CHECK("mlstm_carry");
     if (dtype == AGAVE_F32) {
-        if (vec) launch_read<float, true>(A, C, (float*)out, ldo, max_rows, stream);
-        else launch_read<float, false>(A, C, (float*)out, ldo, max_rows, stream);
+        if (vec) choose_read<float, true>(A, C, (float*)out, ldo, chunks, stream);
+        else choose_read<float, false>(A, C, (float*)out, ldo, chunks, stream);
     } else {
-        if (vec) launch_read<bf16, true>(A, C, (bf16*)out, ldo, max_rows, stream);
-        else launch_read<bf16, false>(A, C, (bf16*)out, ldo, max_rows, stream);
+        if (vec) choose_read<bf16, true>(A, C, (bf16*)out, ldo, chunks, stream);
+        else choose_read<bf16, false>(A, C, (bf16*)out, ldo, chunks, stream);
     }
     AGAVE_LAUNCH_CHECK("mlstm_read");
     return 0;

@@ -293,28 +293,38 @@ def test_linear_with_a_bias_on_every_path(dtype, rows, out_f, in_f, slices_ok):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_gated_ffn_part_with_biases(dtype):
-    """Biases on gate, up and down: the gate/up product then keeps its rows in order (the product
-    that ends in the activation has no place for a bias) and the elementwise kernel follows."""
+@pytest.mark.parametrize("both", [True, False])
+def test_gated_ffn_part_with_biases(dtype, both):
+    """Biases on gate, up and down: on the matrix cores gate's and up's are added inside the product that ends in the
+    activation.  With a bias on one of the two the product keeps its rows in order and the elementwise kernel follows.
+    ``down``'s bias is the part's own unless a caller takes it over."""
     from agave_amd.config.spec import GatedFfnSpec
     from agave_amd.parts import GatedFfn
     hidden, inter = 96, 200
     spec = GatedFfnSpec(kind="gated_dense", hidden=hidden, intermediate=inter, activation="gelu_tanh",
-                        gate_proj="f.g", up_proj="f.u", down_proj="f.d", gate_bias="f.gb", up_bias="f.ub", down_bias="f.db")
+                        gate_proj="f.g", up_proj="f.u", down_proj="f.d", gate_bias="f.gb", up_bias="f.ub" if both else "",
+                        down_bias="f.db")
     t = {"f.g": rnd((inter, hidden), 70, 0.1), "f.u": rnd((inter, hidden), 71, 0.1), "f.d": rnd((hidden, inter), 72, 0.1),
          "f.gb": rnd((inter,), 74, 1.0), "f.ub": rnd((inter,), 75, 1.0), "f.db": rnd((hidden,), 76, 1.0)}
+    if not both:
+        del t["f.ub"]
     b = Bench(dtype)
     needs = GatedFfn.tensor_needs(spec)
     assert {n.name for n in needs} == set(t)
     part = GatedFfn(spec, weights_of(t, needs, dtype), b.env)
-    assert not part.gate_up.interleave_ff
+    assert part.gate_up.interleave_ff == (inter if both and dtype == "bfloat16" else 0)
     for rows in (6, 150):
         x = rnd((rows, hidden), 73, 2.0)
         y = part.forward(x.to(b.dtype).to(DEV), None)
         y = y.sum(0) if y.dim() == 3 else y
         xd = x.to(b.dtype).double()
-        ref = (P.gelu_tanh(xd @ t["f.g"].T + t["f.gb"]) * (xd @ t["f.u"].T + t["f.ub"])) @ t["f.d"].T + t["f.db"]
+        ref = (P.gelu_tanh(xd @ t["f.g"].T + t["f.gb"]) * (xd @ t["f.u"].T + t.get("f.ub", 0.0))) @ t["f.d"].T + t["f.db"]
         check(y, ref, dtype, f"feed-forward with biases, {rows} rows")
+    bias = part.hand_over_bias()
+    assert torch.equal(bias.cpu().double(), t["f.db"].to(b.dtype).double()) and part.hand_over_bias() is None
+    y = part.forward(x.to(b.dtype).to(DEV), None)
+    y = y.sum(0) if y.dim() == 3 else y
+    check(y, ref - t["f.db"], dtype, "without the bias that was handed over")
 
 
 def test_gated_ffn_at_a_prompts_length_comes_in_slices_that_the_residual_kernel_adds():
