@@ -301,10 +301,11 @@ class RglruSpec(MixerSpec):
 
 @dataclass(frozen=True)
 class MlstmSpec(MixerSpec):
-    """The matrix memory of xLSTM (state S [heads, v_head_dim, head_dim], n [heads, head_dim] and m [heads]).
+    """The mLSTM of xLSTM: a matrix per head that is written with exponential gates (state S [heads, v_head_dim, head_dim],
+    n [heads, head_dim] and m [heads]).
 
-    ``q = q_proj x * head_dim^-1/2``, ``k = k_proj x``, ``v = v_proj x``; per head, with cap(z) = gate_cap tanh(z / gate_cap),
-    a log input gate ``i = cap(i_gate x + i_bias)`` and a log forget gate ``f = logsigmoid(cap(f_gate x + f_bias))``;
+    ``q = q_proj x * head_dim^-1/2``, ``k = k_proj x``, ``v = v_proj x``; a head's gates in logarithms, with cap(z) =
+    gate_cap tanh(z / gate_cap), are ``i = cap(i_gate x + i_bias)`` (input) and ``f = logsigmoid(cap(f_gate x + f_bias))`` (forget);
     ``m' = max(f + m, i)`` from m = 0; ``S <- exp(f + m - m') S + exp(i - m') k v^T``, n likewise with k alone;
     ``o = S^T q / (max(|n . q|, exp(-m')) + floor_eps)``; each head's o divided by its root mean square, times ``out_norm``,
     times ``sigmoid(gate_proj x)``; ``o_proj``."""
